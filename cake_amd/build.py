@@ -59,9 +59,12 @@ def _run(cmd: list[str]) -> None:
         raise RuntimeError(f"command failed ({r.returncode}): {' '.join(cmd)}\n{r.stdout}\n{r.stderr}")
 
 
+# packed FP32 math stays off in every HIP object: some v_pk_*_f32 forms the compiler picks by
+# itself have given wrong results now and then on this hardware, with no error
 # per-file hipcc flags: the GEMM's compile-time-unrolled interleaved schedule needs its
 # lambdas fully inlined (below the default threshold the 128x128-per-wave tile keeps
 # closures in scratch memory)
+NO_PK_FP32 = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 HIP_EXTRA = {"gemm": ["-mllvm", "-inline-threshold=100000"]}  # gemm.hip and gemm_inst_*.hip
 
 
@@ -71,7 +74,7 @@ def _compile_hip(src: Path, force: bool) -> Path:
     headers = sorted((CSRC / "kernels").glob("*.h"))
     if force or _newer(src, headers, out):
         _run([HIPCC, "-O3", f"--offload-arch={ARCH}", "-std=c++17", "-fPIC",
-              "-Wno-unused-result", "-munsafe-fp-atomics",
+              "-Wno-unused-result", "-munsafe-fp-atomics", *NO_PK_FP32,
               *HIP_EXTRA.get(src.stem.split("_")[0], []),
               "-c", str(src), "-o", str(out)])
     return out
