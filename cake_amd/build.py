@@ -3,12 +3,16 @@
 Everything is compiled in-tree into ``cake_amd/lib/`` so the shared objects
 travel with the repository snapshot to the GPU box:
 
-* ``libcake_kernels.so`` — every ``csrc/kernels/*.hip`` file, ``hipcc
+* ``libcake_gemm.so`` (``csrc/kernels/gemm*.hip``), ``libcake_mixers.so``
+  (``csrc/kernels/mixer_*.hip``: the hybrid designs' layers) and
+  ``libcake_kernels.so`` (every other ``csrc/kernels/*.hip`` file), ``hipcc
   --offload-arch=gfx950``; plain C ABI (``extern "C" cake_*``) driven from
-  :mod:`cake_amd.ops.hip` through ctypes with torch's current HIP stream, so
-  the launches are capturable in hipGraphs.  Also ``csrc/driver/*.cpp``: the
+  :mod:`cake_amd.ops` through ctypes with torch's current HIP stream, so
+  the launches are capturable in hipGraphs.  ``libcake_kernels.so`` needs
+  ``libcake_gemm.so`` and also holds ``csrc/driver/*.cpp``: the
   native decode loop that replays the captured step graphs
-  (:mod:`cake_amd.runtime.graph_loop`).
+  (:mod:`cake_amd.ops.graph_loop`).  The split lets a program that serves one
+  model compile only what that model runs (:func:`ensure_text`).
 * ``libcake_runtime.so`` — ``csrc/runtime/*.cpp`` (topology parser, wire codec,
   safetensors mmap reader/writer, framed TCP transport), C ABI.
 * ``cake-split-model`` — native executable (``csrc/tools/split_model.cpp``).
@@ -41,6 +45,8 @@ HIPCC = shutil.which("hipcc") or "/opt/rocm/bin/hipcc"
 CXX = shutil.which("g++") or "c++"
 
 KERNEL_LIB = LIB / "libcake_kernels.so"
+GEMM_LIB = LIB / "libcake_gemm.so"
+MIXER_LIB = LIB / "libcake_mixers.so"
 RUNTIME_LIB = LIB / "libcake_runtime.so"
 SPLIT_TOOL = LIB / "cake-split-model"
 CLI_TOOL = LIB / "cake-cli"
@@ -103,26 +109,49 @@ PY_EXT = LIB / "_cake_runtime"  # + EXT_SUFFIX
 EXPERIMENTAL = os.environ.get("CAKE_BUILD_EXPERIMENTAL", "0") != "0"
 
 
-def build_kernels(force: bool = False, jobs: int = 8) -> Path:
-    # HIP kernels + the native graph-replay decode driver (host code on the HIP runtime).
-    # csrc/experimental (the persistent decode engine, measured slower than the launch
-    # path: profiles/r4_mk_summary.md) only with CAKE_BUILD_EXPERIMENTAL=1.
-    srcs = sorted((CSRC / "kernels").glob("*.hip")) + sorted((CSRC / "driver").glob("*.cpp"))
+def _kernel_sources() -> dict[Path, list[Path]]:
+    """Shared object -> its sources.  csrc/experimental (the persistent decode engine,
+    measured slower than the launch path: profiles/r4_mk_summary.md) only with
+    CAKE_BUILD_EXPERIMENTAL=1."""
+    hip = sorted((CSRC / "kernels").glob("*.hip"))
+    gemm = [p for p in hip if p.stem == "gemm" or p.stem.startswith("gemm_inst")]
+    mixers = [p for p in hip if p.stem.startswith("mixer_")]
+    rest = [p for p in hip if p not in gemm and p not in mixers]
+    rest += sorted((CSRC / "driver").glob("*.cpp"))
     if EXPERIMENTAL:
-        srcs += sorted((CSRC / "experimental").glob("*.hip"))
+        rest += sorted((CSRC / "experimental").glob("*.hip"))
+    return {GEMM_LIB: gemm, MIXER_LIB: mixers, KERNEL_LIB: rest}
+
+
+def build_kernels(force: bool = False, jobs: int = 8,
+                  libs: tuple[Path, ...] = (GEMM_LIB, MIXER_LIB, KERNEL_LIB)) -> Path:
+    # HIP kernels + the native graph-replay decode driver (host code on the HIP runtime)
+    groups = {lib: srcs for lib, srcs in _kernel_sources().items() if lib in libs}
+    # the GEMM instantiations compile longest: first in the queue
+    todo = sorted((s for srcs in groups.values() for s in srcs),
+                  key=lambda p: not p.stem.startswith("gemm_inst"))
     with cf.ThreadPoolExecutor(max_workers=jobs) as ex:
-        objs = list(ex.map(lambda s: _compile_hip(s, force), srcs))
+        objs = dict(zip(todo, ex.map(lambda s: _compile_hip(s, force), todo)))
     LIB.mkdir(parents=True, exist_ok=True)
-    stale = [o for o in (BUILD / "kernels").glob("*.o") if o not in objs]
+    keep = {BUILD / "kernels" / (s.stem + ".o")
+            for srcs in _kernel_sources().values() for s in srcs}
+    stale = [o for o in (BUILD / "kernels").glob("*.o") if o not in keep]
     for o in stale:  # an object of a source no longer built (experimental off) must go
         o.unlink()
-    if force or stale or any(_newer(o, [], KERNEL_LIB) for o in objs):
+    for lib, srcs in groups.items():
+        mine = [objs[s] for s in srcs]
         # hipBLASLt for the plain prefill GEMMs it measured faster on (driver/blaslt.cpp);
         # in a torch process the soname resolves to the copy torch already loaded
-        # --no-undefined: a kernel whose host stub the compiler dropped fails here, not at
-        # dlopen on the GPU box
-        _run([HIPCC, f"--offload-arch={ARCH}", "-shared", "-fPIC", *map(str, objs),
-              "-o", str(KERNEL_LIB), "-L/opt/rocm/lib", "-lhipblaslt", "-Wl,--no-undefined"])
+        extra = [] if lib != KERNEL_LIB else [
+            "-L/opt/rocm/lib", "-lhipblaslt", f"-L{LIB}", "-Wl,--no-as-needed", "-lcake_gemm",
+            "-Wl,-rpath,$ORIGIN"]
+        if force or stale or any(_newer(o, [], lib) for o in mine):
+            # --no-undefined: a kernel whose host stub the compiler dropped fails here, not at
+            # dlopen on the GPU box
+            tmp = lib.with_suffix(f".tmp{os.getpid()}")
+            _run([HIPCC, f"--offload-arch={ARCH}", "-shared", "-fPIC", *map(str, mine),
+                  "-o", str(tmp), f"-Wl,-soname,{lib.name}", *extra, "-Wl,--no-undefined"])
+            os.replace(tmp, lib)
     return KERNEL_LIB
 
 
@@ -135,24 +164,33 @@ def _embed_flags() -> tuple[list[str], list[str]]:
     return inc, [f"-L{libdir}", f"-lpython{ver}", "-ldl", "-lm", "-lpthread"]
 
 
-def build_runtime(force: bool = False, jobs: int = 8) -> Path:
-    """C++ host runtime: pybind11 module, C-ABI library, split-model tool and cake-cli."""
+def build_runtime_module(force: bool = False, jobs: int = 8) -> tuple[Path, list[Path]]:
+    """The pybind11 module of the C++ host runtime (safetensors reader, topology, codec)."""
     rt = CSRC / "runtime"
     core_srcs = [rt / f"{n}.cpp" for n in ("json", "topology", "proto", "net", "safetensors",
                                             "server", "native_worker")]
     inc, ext = _py_ext_flags()
-    einc, elink = _embed_flags()
     with cf.ThreadPoolExecutor(max_workers=jobs) as ex:
-        core = list(ex.map(lambda s: _compile_cpp(s, force), core_srcs))
-        capi_f = ex.submit(_compile_cpp, rt / "capi.cpp", force)
         bind_f = ex.submit(_compile_cpp, rt / "bindings.cpp", force, inc)
-        emb_f = ex.submit(_compile_cpp, rt / "embed.cpp", force, einc)
-        capi, bind, emb = capi_f.result(), bind_f.result(), emb_f.result()
+        core = list(ex.map(lambda s: _compile_cpp(s, force), core_srcs))
+        bind = bind_f.result()
     LIB.mkdir(parents=True, exist_ok=True)
     pyext = PY_EXT.with_name(PY_EXT.name + ext)
     if force or any(_newer(o, [], pyext) for o in [*core, bind]):
         _run([CXX, "-shared", "-fPIC", *map(str, core), str(bind), "-o", str(pyext), "-lpthread",
               "-ldl"])
+    return pyext, core
+
+
+def build_runtime(force: bool = False, jobs: int = 8) -> Path:
+    """C++ host runtime: pybind11 module, C-ABI library, split-model tool and cake-cli."""
+    rt = CSRC / "runtime"
+    einc, elink = _embed_flags()
+    pyext, core = build_runtime_module(force, jobs)
+    with cf.ThreadPoolExecutor(max_workers=jobs) as ex:
+        capi_f = ex.submit(_compile_cpp, rt / "capi.cpp", force)
+        emb_f = ex.submit(_compile_cpp, rt / "embed.cpp", force, einc)
+        capi, emb = capi_f.result(), emb_f.result()
     if force or any(_newer(o, [], RUNTIME_LIB) for o in [*core, capi, emb]):
         _run([CXX, "-shared", "-fPIC", *map(str, core), str(capi), str(emb), "-o",
               str(RUNTIME_LIB), *elink])
@@ -189,9 +227,24 @@ def build_engine(force: bool = False) -> Path:
         eng_objs.append(out)
     if force or any(_newer(o, [], ENGINE_LIB) for o in [*eng_objs, *objs, KERNEL_LIB]):
         _run([HIPCC, "-shared", "-fPIC", *map(str, eng_objs), *map(str, objs), "-o",
-              str(ENGINE_LIB), f"-L{LIB}", "-lcake_kernels", "-Wl,-rpath,$ORIGIN",
+              str(ENGINE_LIB), f"-L{LIB}", "-lcake_kernels", "-lcake_gemm", "-Wl,-rpath,$ORIGIN",
               "-Wl,--no-undefined"])
     return ENGINE_LIB
+
+
+def ensure_text(libs: tuple[str, ...], jobs: int | None = None) -> None:
+    """Compile what is missing for a text model run from this checkout: the named kernel
+    libraries ("gemm", "mixers", "kernels") and the runtime module.  Libraries that are
+    there already are used as they are."""
+    jobs = jobs or int(os.environ.get("MAX_JOBS") or min(16, os.cpu_count() or 4))
+    paths = {"gemm": GEMM_LIB, "mixers": MIXER_LIB, "kernels": KERNEL_LIB}
+    need = tuple(paths[n] for n in libs if not paths[n].exists())
+    if KERNEL_LIB in need and not GEMM_LIB.exists() and GEMM_LIB not in need:
+        need = (GEMM_LIB, *need)
+    if not PY_EXT.with_name(PY_EXT.name + _py_ext_flags()[1]).exists():
+        build_runtime_module(jobs=jobs)
+    if need:
+        build_kernels(jobs=jobs, libs=need)
 
 
 def build_all(force: bool = False, jobs: int = 8) -> None:

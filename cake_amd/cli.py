@@ -123,6 +123,9 @@ def _run(args) -> int:
     setup_logging(args.log_level)
     from .context import Context
     ctx = Context.from_args(args)
+    if ctx.model_type == "text-model":
+        from .models.registry import check_placement
+        check_placement(ctx)
     if args.transport == "rccl":
         from .parallel.rccl_roles import run_rccl
         run_rccl(ctx)

@@ -145,10 +145,13 @@ CAKE_API long long cake_gemm_ws_floats(int cfg, int splits, int M, int N, int K,
 // [0, N), up/gate-2 rows [N, 2N)).  splits > 1 needs ws = splits * M * Nv f32.
 // Requirements (host-checked in ops/gemm.py): K % 8 == 0, lda/ldb % 8 == 0,
 // 16-byte aligned operand bases, gated => N % 16 == 0.
-CAKE_API int cake_gemm(int dt, int epi, int cfg, int splits, const void* a, long long lda,
-                       const void* b, long long ldb, void* c, long long ldc, const void* bias,
-                       void* resid, long long ldr, float* ws, const void* zeros, int M, int N,
-                       int K, hipStream_t st) {
+// alpha (f32 epilogues only, 1 elsewhere): r32 (+)= alpha * (x W^T + bias).
+CAKE_API int cake_gemm_scaled(int dt, int epi, int cfg, int splits, const void* a, long long lda,
+                              const void* b, long long ldb, void* c, long long ldc,
+                              const void* bias, void* resid, long long ldr, float* ws,
+                              const void* zeros, int M, int N, int K, float alpha,
+                              hipStream_t st) {
+  if (alpha != 1.f && epi != kEpiResid32 && epi != kEpiStore32) return (int)hipErrorInvalidValue;
   int act = 0;
   if (epi == 8 || epi == 9) {  // quick_gelu / GELU: the activation epilogue, other act
     act = epi - 7;
@@ -177,6 +180,7 @@ CAKE_API int cake_gemm(int dt, int epi, int cfg, int splits, const void* a, long
   g.M = M; g.N = N; g.K = K;
   g.gated = gated ? 1 : 0;
   g.act = act;
+  g.alpha = alpha;
   g.half = N;
   g.Nv = gated ? 2 * N : N;
   g.tiles_m = (M + bm - 1) / bm;
@@ -208,4 +212,12 @@ CAKE_API int cake_gemm(int dt, int epi, int cfg, int splits, const void* a, long
   const dim3 fgrid((N + 1023) / 1024, M);
   return (dt == kBF16) ? dispatch_finalize<kBF16>(epi, fgrid, st, g, splits)
                        : dispatch_finalize<kF16>(epi, fgrid, st, g, splits);
+}
+
+CAKE_API int cake_gemm(int dt, int epi, int cfg, int splits, const void* a, long long lda,
+                       const void* b, long long ldb, void* c, long long ldc, const void* bias,
+                       void* resid, long long ldr, float* ws, const void* zeros, int M, int N,
+                       int K, hipStream_t st) {
+  return cake_gemm_scaled(dt, epi, cfg, splits, a, lda, b, ldb, c, ldc, bias, resid, ldr, ws,
+                          zeros, M, N, K, 1.f, st);
 }

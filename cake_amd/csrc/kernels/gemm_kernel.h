@@ -46,6 +46,7 @@ struct GemmArgs {
   int gated;             // B row order interleaves 16-row blocks of two halves
   int tiles_m, tiles_n, kps;  // k elements per split
   int act;               // kEpiSilu activation: 0 SiLU, 1 quick_gelu, 2 GELU (erf)
+  float alpha = 1.f;     // kEpiResid32 / kEpiStore32: factor of the product (and bias)
   // in-kernel split-K pair (gemm_4w.h, splits == 2): the first split of a tile to finish
   // parks its accumulators in ws (one 256x256 f32 slab per tile), the second adds them and
   // runs the epilogue; tick = [kPairTiles arrival counters | kPairTiles ready flags]
@@ -306,12 +307,13 @@ __device__ __forceinline__ void epi_strip(const GemmArgs& g, const cf32x4 (&tile
 #pragma unroll
             for (int c = 0; c < CPL; c += 4) {
               float4 o = ADD ? *reinterpret_cast<float4*>(r + c) : make_float4(0.f, 0.f, 0.f, 0.f);
-              o.x += v[c]; o.y += v[c + 1]; o.z += v[c + 2]; o.w += v[c + 3];
+              o.x = fmaf(g.alpha, v[c], o.x); o.y = fmaf(g.alpha, v[c + 1], o.y);
+              o.z = fmaf(g.alpha, v[c + 2], o.z); o.w = fmaf(g.alpha, v[c + 3], o.w);
               *reinterpret_cast<float4*>(r + c) = o;
             }
           } else {
             for (int c = 0; c < CPL; ++c)
-              if (n0c + c < g.N) r[c] = ADD ? r[c] + v[c] : v[c];
+              if (n0c + c < g.N) r[c] = fmaf(g.alpha, v[c], ADD ? r[c] : 0.f);
           }
         } else {
           if constexpr (EPI == kEpiAdd16) {
@@ -510,12 +512,13 @@ __device__ __forceinline__ void readout_strip_w(const GemmArgs& g, const float* 
         float* r = g.r32 + (size_t)m * g.ldr + n;
         if (n + 4 <= g.N && ((g.ldr | n) & 3) == 0) {
           float4 o = R32 ? rold[R32 ? p : 0][R32 ? c : 0] : make_float4(0.f, 0.f, 0.f, 0.f);
-          o.x += v[0]; o.y += v[1]; o.z += v[2]; o.w += v[3];
+          o.x = fmaf(g.alpha, v[0], o.x); o.y = fmaf(g.alpha, v[1], o.y);
+          o.z = fmaf(g.alpha, v[2], o.z); o.w = fmaf(g.alpha, v[3], o.w);
           *reinterpret_cast<float4*>(r) = o;
         } else {
           constexpr bool ADD = R32;
           for (int e = 0; e < 4; ++e)
-            if (n + e < g.N) r[e] = ADD ? r[e] + v[e] : v[e];
+            if (n + e < g.N) r[e] = fmaf(g.alpha, v[e], ADD ? r[e] : 0.f);
         }
       } else {
         const int n = vcol0 + lc;
@@ -867,8 +870,10 @@ __global__ __launch_bounds__(256) void gemm_splitk_finalize(GemmArgs g, int spli
       if constexpr (EPI == kEpiAdd16) y += to_f32<DT>(g.r16[(size_t)m * g.ldr + fq]);
       if constexpr (EPI == kEpiSilu) y = gemm_act(g.act, y);
     }
-    if constexpr (EPI == kEpiResid32) g.r32[(size_t)m * g.ldr + fq] += y;
-    else if constexpr (EPI == kEpiStore32) g.r32[(size_t)m * g.ldr + fq] = y;
+    if constexpr (EPI == kEpiResid32) {
+      float* r = g.r32 + (size_t)m * g.ldr + fq;
+      *r = fmaf(g.alpha, y, *r);
+    } else if constexpr (EPI == kEpiStore32) g.r32[(size_t)m * g.ldr + fq] = g.alpha * y;
     else g.c[(size_t)m * g.ldc + fq] = from_f32<DT>(y);
   }
 }

@@ -2,18 +2,18 @@
 // tail (lm_head + repeat penalty + argmax + step finalize).  Kernels: gemv_kernel.h.
 #include "gemv_kernel.h"
 
-template <bool SEL>
+template <bool SEL, bool OFF = false>
 static int launch_norm_f32(int dt, const float* resid, const void* norm_w, float eps,
                            const void* w, int K, int N, float* out, const HeadSel& hs,
-                           hipStream_t st) {
-  if (K % 8) return (int)hipErrorInvalidValue;
+                           hipStream_t st, int Kn = 0, float off = 0.f) {
+  if (K % 8 || Kn < 0 || Kn > K) return (int)hipErrorInvalidValue;
   const size_t lds = (size_t)K * sizeof(float);
   const GemvTune t = g_tune[kNormF32];
-  DISPATCH_DT(dt, DISPATCH_TUNE(t, K, CAKE_NX_NORM(K, hipLaunchKernelGGL((gemv_norm_f32_kernel<DT, U, PF, NX, SEL>),
+  DISPATCH_DT(dt, DISPATCH_TUNE(t, K, CAKE_NX_NORM(K, hipLaunchKernelGGL((gemv_norm_f32_kernel<DT, U, PF, NX, SEL, OFF>),
                                                       dim3(grid_for((N + 1) / 2, t.MB)),
                                                       dim3(kGemvThreads), lds, st, resid,
                                                       (const uint16_t*)norm_w, eps,
-                                                      (const uint16_t*)w, K, N, out, hs))));
+                                                      (const uint16_t*)w, K, N, out, hs, Kn, off))));
   return (int)hipGetLastError();
 }
 
@@ -37,4 +37,27 @@ CAKE_API int cake_head_select(int dt, const float* resid, const void* norm_w, fl
   const HeadSel hs{hist, hist_len, last_n, penalty, slot, ticket, tok, hist, hist_len, pos,
                    max_hist, (const uint16_t*)embed, emb_out, K};
   return launch_norm_f32<true>(dt, resid, norm_w, eps, w, K, N, out, hs, st);
+}
+
+// The same pair for a norm weight stored around `off` and a row of Kn <= K values (zeros up
+// to K).
+CAKE_API int cake_gemv_norm_f32_off(int dt, const float* resid, const void* norm_w, float eps,
+                                    float off, int Kn, const void* w, int K, int N, float* out,
+                                    hipStream_t st) {
+  if (Kn < 1) return (int)hipErrorInvalidValue;
+  return launch_norm_f32<false, true>(dt, resid, norm_w, eps, w, K, N, out, HeadSel{}, st, Kn, off);
+}
+
+CAKE_API int cake_head_select_off(int dt, const float* resid, const void* norm_w, float eps,
+                                  float off, int Kn, const void* w, int K, int N, float* out,
+                                  int* hist, int* hist_len, int last_n, float penalty,
+                                  unsigned long long* slot, unsigned int* ticket, int* tok,
+                                  int* pos, int max_hist, const void* embed, float* emb_out,
+                                  hipStream_t st) {
+  if (last_n < 0 || last_n > 256 || !(penalty > 0.f) || slot == nullptr || ticket == nullptr ||
+      Kn < 1 || (embed != nullptr && (emb_out == nullptr || K % 8)))
+    return (int)hipErrorInvalidValue;
+  const HeadSel hs{hist, hist_len, last_n, penalty, slot, ticket, tok, hist, hist_len, pos,
+                   max_hist, (const uint16_t*)embed, emb_out, K};
+  return launch_norm_f32<true, true>(dt, resid, norm_w, eps, w, K, N, out, hs, st, Kn, off);
 }

@@ -40,6 +40,33 @@ __device__ __forceinline__ void stage_rmsnorm(const float* __restrict__ x,
   __syncthreads();
 }
 
+// The same for a weight stored around `off` (off + w), the mean over the first Kn <= K
+// columns (columns past Kn hold zeros).
+template <int DT>
+__device__ __forceinline__ void stage_rmsnorm_off(const float* __restrict__ x,
+                                                  const uint16_t* __restrict__ w, float eps,
+                                                  int K, int Kn, float off, float* xs) {
+  __shared__ float red[16];
+  float ss = 0.f;
+  for (int i = threadIdx.x * 4; i < K; i += kGemvThreads * 4) {
+    const float4 v = *reinterpret_cast<const float4*>(x + i);
+    *reinterpret_cast<float4*>(xs + i) = v;
+    ss += v.x * v.x + v.y * v.y + v.z * v.z + v.w * v.w;
+  }
+  ss = block_sum(ss, red);
+  const float r = rsqrtf(ss / (float)Kn + eps);
+  for (int i = threadIdx.x * 4; i < K; i += kGemvThreads * 4) {
+    float4 v = *reinterpret_cast<const float4*>(xs + i);
+    const uint2 wv = *reinterpret_cast<const uint2*>(w + i);
+    v.x *= r * (off + to_f32<DT>((uint16_t)(wv.x & 0xffff)));
+    v.y *= r * (off + to_f32<DT>((uint16_t)(wv.x >> 16)));
+    v.z *= r * (off + to_f32<DT>((uint16_t)(wv.y & 0xffff)));
+    v.w *= r * (off + to_f32<DT>((uint16_t)(wv.y >> 16)));
+    *reinterpret_cast<float4*>(xs + i) = v;
+  }
+  __syncthreads();
+}
+
 // Copy a 16-bit activation row into LDS (kept 16-bit: 70B down_proj has K=28672).
 __device__ __forceinline__ void stage_plain16(const uint16_t* __restrict__ x, int K,
                                               uint16_t* xs) {
@@ -81,6 +108,26 @@ template <int DT, int NX> struct NormPre {  // K <= 1024 NX, K % 4 == 0
       v.y *= r * to_f32<DT>((uint16_t)(w[j].x >> 16));
       v.z *= r * to_f32<DT>((uint16_t)(w[j].y & 0xffff));
       v.w *= r * to_f32<DT>((uint16_t)(w[j].y >> 16));
+      if (i < K) *reinterpret_cast<float4*>(xs + i) = v;
+    }
+    __syncthreads();
+  }
+  // weight stored around `off`, the mean over Kn <= K columns (zeros past Kn)
+  __device__ __forceinline__ void finish_off(float eps, int K, int Kn, float off, float* xs) {
+    __shared__ float red[16];
+    float ss = 0.f;
+#pragma unroll
+    for (int j = 0; j < NX; ++j) ss += x[j].x * x[j].x + x[j].y * x[j].y + x[j].z * x[j].z + x[j].w * x[j].w;
+    ss = block_sum(ss, red);
+    const float r = rsqrtf(ss / (float)Kn + eps);
+#pragma unroll
+    for (int j = 0; j < NX; ++j) {
+      const int i = (j * kGemvThreads + threadIdx.x) * 4;
+      float4 v = x[j];
+      v.x *= r * (off + to_f32<DT>((uint16_t)(w[j].x & 0xffff)));
+      v.y *= r * (off + to_f32<DT>((uint16_t)(w[j].x >> 16)));
+      v.z *= r * (off + to_f32<DT>((uint16_t)(w[j].y & 0xffff)));
+      v.w *= r * (off + to_f32<DT>((uint16_t)(w[j].y >> 16)));
       if (i < K) *reinterpret_cast<float4*>(xs + i) = v;
     }
     __syncthreads();
@@ -414,10 +461,12 @@ __device__ __forceinline__ unsigned int ordered_key(float f) {
 }
 
 // RMSNorm(f32 row) then f32 output: the lm_head (SEL: + greedy selection, see HeadSel).
-template <int DT, int U, int PFC, int NX, bool SEL>
+// OFF: a norm weight stored around `off`, the mean over Kn <= K columns.
+template <int DT, int U, int PFC, int NX, bool SEL, bool OFF>
 __global__ __launch_bounds__(kGemvThreads) void gemv_norm_f32_kernel(
     const float* __restrict__ resid, const uint16_t* __restrict__ norm_w, float eps,
-    const uint16_t* __restrict__ w, int K, int N, float* __restrict__ out, HeadSel hs) {
+    const uint16_t* __restrict__ w, int K, int N, float* __restrict__ out, HeadSel hs, int Kn,
+    float off) {
   extern __shared__ float xs[];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int npairs = (N + 1) >> 1;
@@ -439,8 +488,13 @@ __global__ __launch_bounds__(kGemvThreads) void gemv_norm_f32_kernel(
   __builtin_amdgcn_sched_barrier(0);  // x loads strictly before the weights (in-order vmcnt)
   if (NX > 0 || (PFC > 0 && p0 < npairs)) prefetch_rows<PFC>(wa0, wb0, pre);  // NX: exact vmcnt
   __builtin_amdgcn_sched_barrier(0);
-  if constexpr (NX > 0) xp.finish(eps, K, xs);
-  else stage_rmsnorm<DT>(resid, norm_w, eps, K, xs);
+  if constexpr (OFF) {
+    if constexpr (NX > 0) xp.finish_off(eps, K, Kn, off, xs);
+    else stage_rmsnorm_off<DT>(resid, norm_w, eps, K, Kn, off, xs);
+  } else {
+    if constexpr (NX > 0) xp.finish(eps, K, xs);
+    else stage_rmsnorm<DT>(resid, norm_w, eps, K, xs);
+  }
   int win[4] = {-1, -1, -1, -1};
   if constexpr (SEL) {
     const int n = min(hs.last_n, hlen), start = hlen - n;

@@ -1,0 +1,701 @@
+// Softmax attention of the hybrid designs: separate query/key and value head sizes,
+// interleaved partial rotary positions, RMS-normalised queries and keys, an optional sink
+// (one extra exp(0) in the denominator) and an optional sigmoid output gate.
+//
+// Cache of one layer run: K [slot][G][S][DP] row-major and V TRANSPOSED [slot][G][DVP][S]
+// (DP = key size padded to 32, DVP = value size padded to 16, zero-filled): both products
+// of both kernels then take 16-byte / 8-byte pieces of contiguous memory as their MFMA
+// operands, and no kernel transposes values in LDS.
+//
+//   * mixer_prep_qk / mixer_prep_v: prompt rows — rotation + norm of q and k, cache write.
+//   * mixer_flash: prompt attention over a ragged batch.  S^T = K Q^T and O^T += V^T P^T
+//     (an accumulator of the first is the B operand of the second), 4 waves x 32 query
+//     rows, key tiles staged in LDS (double-buffered, next tile's loads in flight behind
+//     the MFMAs), gate and head concatenation in the epilogue.
+//   * mixer_attn_decode: one token per sequence — rotation, norm and cache write of the new
+//     key/value in the prologue, K / V^T streamed straight from memory into MFMA operands,
+//     split over the keys with an in-launch merge, gate in the epilogue.
+#include "mixer_common.h"
+
+namespace cake {
+
+// ---------------------------------------------------------------------------
+// prompt rows: q, k -> rotated, normalised
+// ---------------------------------------------------------------------------
+struct PrepArgs {
+  const void* proj;      // [N][ldp] q | k | v | ... columns
+  long long ldp;
+  int N, H, G, dim, vdim, DP, DVP, S, rd2;  // rd2 = rotated pairs
+  int qk_norm;
+  float eps;
+  const float2* cs;      // [positions][rd2] (cos, sin)
+  const int* row_pos;    // [N]
+  const int* row_slot;   // [N]
+  void* qn;              // [N][H][DP]
+  void* kc;              // layer run's K cache
+  void* vc;              // layer run's V^T cache
+  long long k_slot, v_slot;  // elements per slot
+};
+
+// LPH lanes per (row, head), four consecutive dims each
+template <int DT>
+__global__ __launch_bounds__(256) void mixer_prep_qk_kernel(PrepArgs a, int lph) {
+  using E = typename St<DT>::E;
+  const int per = 256 / lph;  // (row, head) items per workgroup
+  const int item = blockIdx.x * per + threadIdx.x / lph;
+  const int l = threadIdx.x % lph, d0 = 4 * l;
+  const int nh = a.H + a.G;
+  if (item >= a.N * nh) return;  // whole lph-lane groups leave together
+  const int n = item / nh, hh = item - n * nh;
+  const bool isq = hh < a.H;
+  const int pos = a.row_pos[n];
+  const E* src = reinterpret_cast<const E*>(a.proj) + (long long)n * a.ldp + (long long)hh * a.dim;
+  float x[4];
+#pragma unroll
+  for (int e = 0; e < 4; ++e) x[e] = d0 + e < a.dim ? St<DT>::ld(src[d0 + e]) : 0.f;
+#pragma unroll
+  for (int p = 0; p < 2; ++p) {
+    const int i = 2 * l + p;
+    if (i < a.rd2) {
+      const float2 t = a.cs[(long long)pos * a.rd2 + i];
+      const float u = x[2 * p], v = x[2 * p + 1];
+      x[2 * p] = u * t.x - v * t.y;
+      x[2 * p + 1] = v * t.x + u * t.y;
+    }
+  }
+  if (a.qk_norm) {
+    float ss = x[0] * x[0] + x[1] * x[1] + x[2] * x[2] + x[3] * x[3];
+    for (int o = lph >> 1; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
+    const float r = 1.f / sqrtf(ss / (float)a.dim + a.eps);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) x[e] *= r;
+  }
+  E* dst = isq ? reinterpret_cast<E*>(a.qn) + ((long long)n * a.H + hh) * a.DP
+               : reinterpret_cast<E*>(a.kc) + a.row_slot[n] * a.k_slot +
+                     ((long long)(hh - a.H) * a.S + pos) * a.DP;
+  if (d0 < a.DP) {  // DP % 4 == 0; columns past dim carry zeros
+    if constexpr (DT == kF32) {
+      *reinterpret_cast<float4*>(dst + d0) = make_float4(x[0], x[1], x[2], x[3]);
+    } else {
+      const uint32_t lo = (uint32_t)St<DT>::st(x[0]) | ((uint32_t)St<DT>::st(x[1]) << 16);
+      const uint32_t hi = (uint32_t)St<DT>::st(x[2]) | ((uint32_t)St<DT>::st(x[3]) << 16);
+      *reinterpret_cast<uint2*>(dst + d0) = make_uint2(lo, hi);
+    }
+  }
+}
+
+// values -> V^T: a wave takes 64 rows x 8 dims, so its stores run along the positions
+template <int DT>
+__global__ __launch_bounds__(256) void mixer_prep_v_kernel(PrepArgs a) {
+  using E = typename St<DT>::E;
+  const int n = blockIdx.x * 64 + (threadIdx.x & 63);
+  const int nch = (a.vdim + 7) / 8;
+  const int c = blockIdx.y * 4 + (threadIdx.x >> 6);
+  if (n >= a.N || c >= a.G * nch) return;
+  const int gh = c / nch, d0 = (c - gh * nch) * 8;
+  const E* src = reinterpret_cast<const E*>(a.proj) + (long long)n * a.ldp +
+                 (long long)(a.H + a.G) * a.dim + (long long)gh * a.vdim + d0;
+  E* dst = reinterpret_cast<E*>(a.vc) + a.row_slot[n] * a.v_slot +
+           ((long long)gh * a.DVP + d0) * a.S + a.row_pos[n];
+#pragma unroll
+  for (int e = 0; e < 8; ++e)
+    if (d0 + e < a.vdim) dst[(long long)e * a.S] = src[e];
+}
+
+// ---------------------------------------------------------------------------
+// prompt attention
+// ---------------------------------------------------------------------------
+struct MixFlashArgs {
+  const void* qn;        // [N][H][DP]
+  const void* kc;
+  const void* vc;
+  long long k_slot, v_slot;
+  const SeqRow* seq;     // [B]
+  const void* gate;      // [N][ldg] + column 0 of the gate (null: no gate)
+  long long ldg;
+  void* out;             // [N][ldo]
+  long long ldo;
+  int H, G, DP, DVP, vdim, S, sink;
+  float scale_log2;
+};
+
+template <int DT, int CLS, bool EXACT>
+__global__ __launch_bounds__(256, CLS <= 128 ? 2 : 1) void mixer_flash_kernel(MixFlashArgs a) {
+  using E = typename St<DT>::E;
+  constexpr int EPC = St<DT>::EPC;
+  constexpr int NKS = CLS / St<DT>::KSTEP, NVT = CLS / 16;
+  constexpr int BN = DT == kF32 ? 32 : 64, NB = BN / 16;  // keys, 16-key blocks per tile
+  constexpr int NPT = CLS / 32;                            // 16-byte pieces per thread, K or V
+  constexpr int NBUF = CLS <= 128 ? 2 : 1;
+  constexpr int VLD = BN + EPC;                            // V^T row stride in LDS
+  constexpr int VPR = BN / EPC;                            // pieces per V^T row
+  extern __shared__ __attribute__((aligned(16))) unsigned char mixer_smem[];
+  E* const sm = reinterpret_cast<E*>(mixer_smem);
+  const int DP = EXACT ? CLS : a.DP, DVP = EXACT ? CLS : a.DVP;
+  const int KLD = DP + EPC;                                // +16 bytes: no bank conflicts
+  const int KPR = DP / EPC;
+  const int bufe = BN * KLD + DVP * VLD;
+  const int nks = EXACT ? NKS : DP / St<DT>::KSTEP, nvt = EXACT ? NVT : DVP / 16;
+
+  const SeqRow sq = a.seq[blockIdx.z];
+  const int nqt = (sq.len + 127) / 128;
+  if ((int)blockIdx.x >= nqt) return;
+  const int m0 = (nqt - 1 - (int)blockIdx.x) * 128;  // the longest rows first
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, l15 = lane & 15, g = lane >> 4;
+  const int h = blockIdx.y, hk = h / (a.H / a.G);
+  const E* kb = reinterpret_cast<const E*>(a.kc) + sq.slot * a.k_slot + (long long)hk * a.S * a.DP;
+  const E* vb = reinterpret_cast<const E*>(a.vc) + sq.slot * a.v_slot + (long long)hk * a.DVP * a.S;
+  const int qw = m0 + wave * 32;  // this wave's first row
+
+  uint4 qf[2][NKS];
+#pragma unroll
+  for (int j = 0; j < 2; ++j) {
+    const int row = min(qw + 16 * j + l15, sq.len - 1);
+    const E* qp = reinterpret_cast<const E*>(a.qn) + ((long long)(sq.row0 + row) * a.H + h) * DP;
+#pragma unroll
+    for (int ks = 0; ks < NKS; ++ks)
+      qf[j][ks] = (EXACT || ks < nks) ? *reinterpret_cast<const uint4*>(qp + (ks * 4 + g) * EPC)
+                                      : make_uint4(0, 0, 0, 0);
+  }
+  cf32x4 o[2][NVT];
+#pragma unroll
+  for (int j = 0; j < 2; ++j)
+#pragma unroll
+    for (int t = 0; t < NVT; ++t) o[j][t] = cf32x4{0.f, 0.f, 0.f, 0.f};
+  // running max (log2 units) and lane-partial sum; the sink is a key of score 0 without value
+  float m[2], l[2];
+#pragma unroll
+  for (int j = 0; j < 2; ++j) {
+    m[j] = a.sink ? 0.f : -INFINITY;
+    l[j] = a.sink && g == 0 ? 1.f : 0.f;
+  }
+  const int kend = min(sq.pos0 + sq.len, sq.pos0 + m0 + 128);
+  const int ntiles = (kend + BN - 1) / BN;
+  const int qmin = sq.pos0 + qw, qmax = qmin + 31;
+
+  u32x4 kr[NPT], vr[NPT];
+  auto gload = [&](int j) __attribute__((always_inline)) {
+#pragma unroll
+    for (int i = 0; i < NPT; ++i) {
+      const int p = tid + 256 * i;
+      if (EXACT || p < BN * KPR)
+        kr[i] = *reinterpret_cast<const u32x4*>(kb + (long long)j * BN * DP + (long long)p * EPC);
+      if (EXACT || p < DVP * VPR) {
+        const int r = p / VPR, c = p - r * VPR;
+        vr[i] = *reinterpret_cast<const u32x4*>(vb + (long long)r * a.S + j * BN + c * EPC);
+      }
+    }
+  };
+  auto sstore = [&](int buf) __attribute__((always_inline)) {
+    E* Ks = sm + buf * bufe;
+    E* Vs = Ks + BN * KLD;
+#pragma unroll
+    for (int i = 0; i < NPT; ++i) {
+      const int p = tid + 256 * i;
+      if (EXACT || p < BN * KPR) {
+        const int r = p / KPR, c = p - r * KPR;
+        *reinterpret_cast<u32x4*>(Ks + r * KLD + c * EPC) = kr[i];
+      }
+      if (EXACT || p < DVP * VPR) {
+        const int r = p / VPR, c = p - r * VPR;
+        *reinterpret_cast<u32x4*>(Vs + r * VLD + c * EPC) = vr[i];
+      }
+    }
+  };
+
+  gload(0);
+  sstore(0);
+  __syncthreads();
+  for (int j = 0; j < ntiles; ++j) {
+    const int buf = NBUF == 2 ? (j & 1) : 0;
+    const bool more = j + 1 < ntiles;
+    const E* Ks = sm + buf * bufe;
+    const E* Vs = Ks + BN * KLD;
+    const int k0 = j * BN;
+    const bool active = k0 <= qmax;  // wave-uniform: some row of this wave sees the tile
+    cf32x4 s[2][NB];
+    if (active) {
+#pragma unroll
+      for (int b = 0; b < NB; ++b) {
+        s[0][b] = cf32x4{0.f, 0.f, 0.f, 0.f};
+        s[1][b] = cf32x4{0.f, 0.f, 0.f, 0.f};
+        const E* krow = Ks + (16 * b + l15) * KLD + g * EPC;
+#pragma unroll
+        for (int ks = 0; ks < NKS; ++ks) {
+          if (EXACT || ks < nks) {
+            const uint4 kf = *reinterpret_cast<const uint4*>(krow + ks * 4 * EPC);
+            s[0][b] = mm_piece<DT>(kf, qf[0][ks], s[0][b]);
+            s[1][b] = mm_piece<DT>(kf, qf[1][ks], s[1][b]);
+          }
+        }
+      }
+    }
+    if (more) gload(j + 1);  // behind the QK products, in flight over the rest of the tile
+    if (active) {
+      const bool edge = k0 + BN - 1 > qmin;
+      PFrag<DT> pf[2][NB / 2];
+#pragma unroll
+      for (int q = 0; q < 2; ++q) {
+        if (edge) {
+          const int qpos = qmin + 16 * q + l15;
+#pragma unroll
+          for (int b = 0; b < NB; ++b)
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+              if (k0 + 16 * b + 4 * g + e > qpos) s[q][b][e] = -INFINITY;
+        }
+        float mx = -INFINITY;
+#pragma unroll
+        for (int b = 0; b < NB; ++b)
+#pragma unroll
+          for (int e = 0; e < 4; ++e) mx = fmaxf(mx, s[q][b][e]);
+        mx = group_max(mx) * a.scale_log2;
+        if (a.scale_log2 < 0.f) {  // a negative scale turns the order round
+          float mn = INFINITY;
+#pragma unroll
+          for (int b = 0; b < NB; ++b)
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+              if (s[q][b][e] != -INFINITY) mn = fminf(mn, s[q][b][e]);
+          mx = group_max(mn == INFINITY ? -INFINITY : mn * a.scale_log2);
+        }
+        const bool grow = mx > m[q];
+        if (__builtin_amdgcn_ballot_w64(grow) != 0ull) {
+          const float mn = fmaxf(m[q], mx);
+          const float alpha = mn == -INFINITY ? 1.f : __builtin_amdgcn_exp2f(m[q] - mn);
+          m[q] = mn;
+          l[q] *= alpha;
+#pragma unroll
+          for (int t = 0; t < NVT; ++t)
+            if (EXACT || t < nvt) o[q][t] *= alpha;
+        }
+        const float mc = m[q] == -INFINITY ? 0.f : m[q];
+        float rs = 0.f;
+#pragma unroll
+        for (int b = 0; b < NB; ++b)
+#pragma unroll
+          for (int e = 0; e < 4; ++e) {
+            const float raw = s[q][b][e];
+            const float p = raw == -INFINITY ? 0.f
+                                             : __builtin_amdgcn_exp2f(fmaf(raw, a.scale_log2, -mc));
+            s[q][b][e] = p;
+            rs += p;
+          }
+        l[q] += rs;
+#pragma unroll
+        for (int b = 0; b < NB / 2; ++b) pf[q][b] = pack_p<DT>(s[q][2 * b], s[q][2 * b + 1]);
+      }
+#pragma unroll
+      for (int b = 0; b < NB / 2; ++b)
+#pragma unroll
+        for (int t = 0; t < NVT; ++t)
+          if (EXACT || t < nvt) {
+            const VFrag<DT> vf = load_v<DT>(Vs + (16 * t + l15) * VLD + 32 * b, g);
+            o[0][t] = mm_pv<DT>(vf, pf[0][b], o[0][t]);
+            o[1][t] = mm_pv<DT>(vf, pf[1][b], o[1][t]);
+          }
+    }
+    if (NBUF == 1) __syncthreads();  // every wave is past the tile before it is replaced
+    if (more) sstore(NBUF == 2 ? buf ^ 1 : 0);
+    __syncthreads();
+  }
+
+  // epilogue: lane (l15, g) holds O^T[16 t + 4 g + e][row l15]
+#pragma unroll
+  for (int j = 0; j < 2; ++j) {
+    const int row = qw + 16 * j + l15;
+    const float lt = group_sum(l[j]);
+    if (row >= sq.len) continue;
+    const float inv = 1.f / lt;
+    const long long n = sq.row0 + row;
+    E* op = reinterpret_cast<E*>(a.out) + n * a.ldo + (long long)h * a.vdim;
+    const E* gp = a.gate ? reinterpret_cast<const E*>(a.gate) + n * a.ldg + (long long)h * a.vdim
+                         : nullptr;
+#pragma unroll
+    for (int t = 0; t < NVT; ++t)
+      if (EXACT || t < nvt) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const int d = 16 * t + 4 * g + e;
+          if (d < a.vdim) {
+            float y = o[j][t][e] * inv;
+            if (gp) y *= sigmoid32(St<DT>::ld(gp[d]));
+            op[d] = St<DT>::st(y);
+          }
+        }
+      }
+  }
+}
+
+// ---------------------------------------------------------------------------
+// decode attention (one token per sequence)
+// ---------------------------------------------------------------------------
+struct MixDecArgs {
+  const float* proj;     // [B][ldp] f32: q | k | v | gate columns
+  long long ldp;
+  const int* pos;        // [B]
+  const int* slot;       // [B]
+  const float2* cs;
+  int rd2, qk_norm, sink, gated;
+  float eps, scale_log2;
+  void* kc;
+  void* vc;
+  long long k_slot, v_slot;
+  void* out;             // [B][ldo]
+  long long ldo;
+  int H, G, dim, vdim, DP, DVP, S, nsplit;
+  float* part;           // [B][ngt][nsplit][16][DVP + 2]
+  unsigned int* ticket;  // [B][ngt], zero between launches
+};
+
+constexpr int kDecWaves = 4;
+
+// rotation + norm of one head by one wave: lane handles dims 4 lane .. +3 (dim <= 256)
+__device__ __forceinline__ void head_rot_norm(const float* src, int dim, int lane,
+                                              const float2* cs, int rd2, int qk_norm, float eps,
+                                              float* x) {
+  const int d0 = 4 * lane;
+#pragma unroll
+  for (int e = 0; e < 4; ++e) x[e] = d0 + e < dim ? src[d0 + e] : 0.f;
+#pragma unroll
+  for (int p = 0; p < 2; ++p) {
+    const int i = 2 * lane + p;
+    if (i < rd2) {
+      const float2 t = cs[i];
+      const float u = x[2 * p], v = x[2 * p + 1];
+      x[2 * p] = u * t.x - v * t.y;
+      x[2 * p + 1] = v * t.x + u * t.y;
+    }
+  }
+  if (qk_norm) {
+    const float ss = wave_sum(x[0] * x[0] + x[1] * x[1] + x[2] * x[2] + x[3] * x[3]);
+    const float r = 1.f / sqrtf(ss / (float)dim + eps);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) x[e] *= r;
+  }
+}
+
+template <int DT, int CLS, bool EXACT>
+__global__ __launch_bounds__(64 * kDecWaves) void mixer_attn_decode_kernel(MixDecArgs a) {
+  using E = typename St<DT>::E;
+  constexpr int EPC = St<DT>::EPC;
+  constexpr int NKS = CLS / St<DT>::KSTEP, NVT = CLS / 16;
+  constexpr bool kPrefetch = DT != kF32 && CLS <= 128;
+  const int DP = EXACT ? CLS : a.DP, DVP = EXACT ? CLS : a.DVP;
+  const int nks = EXACT ? NKS : DP / St<DT>::KSTEP, nvt = EXACT ? NVT : DVP / 16;
+  __shared__ __attribute__((aligned(16))) E qs[16 * (CLS + EPC)];
+  __shared__ __attribute__((aligned(16))) E kcur[CLS];
+  __shared__ __attribute__((aligned(16))) E vcur[CLS];
+  __shared__ float red_m[kDecWaves][16], red_l[kDecWaves][16];
+  __shared__ float red_o[kDecWaves][16][CLS + 1];
+  __shared__ int s_last;
+
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, l15 = lane & 15, g = lane >> 4;
+  const int R = a.H / a.G, npg = (R + 15) / 16;      // 16-row query tiles per kv head
+  const int gt = blockIdx.x, hk = gt / npg, r0 = (gt - hk * npg) * 16;
+  const int nr = min(16, R - r0);
+  const int sp = blockIdx.y, b = blockIdx.z;
+  const int pos = a.pos[b], slot = a.slot[b];
+  // key split: multiples of 128 keys, the last active one owns the new key
+  const int Tk = pos + 1;
+  const int kps = ((Tk + a.nsplit - 1) / a.nsplit + 127) / 128 * 128;
+  const int nact = (Tk + kps - 1) / kps;
+  if (sp >= nact) return;
+  const bool owner = sp == nact - 1;
+  const int kbeg = sp * kps, klim = min(kbeg + kps, pos);  // cached keys [kbeg, klim)
+  const float* pj = a.proj + (long long)b * a.ldp;
+  const float2* cs = a.cs + (long long)pos * a.rd2;
+  E* kb = reinterpret_cast<E*>(a.kc) + slot * a.k_slot + (long long)hk * a.S * a.DP;
+  E* vb = reinterpret_cast<E*>(a.vc) + slot * a.v_slot + (long long)hk * a.DVP * a.S;
+
+  // the wave's first block of keys is requested ahead of the prologue
+  uint4 kf[2][NKS];
+  VFrag<DT> vf[NVT];
+  auto load_k = [&](int k0) {
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+      const E* kp = kb + (long long)(k0 + 16 * u + l15) * DP + g * EPC;
+#pragma unroll
+      for (int ks = 0; ks < NKS; ++ks)
+        if (EXACT || ks < nks) kf[u][ks] = *reinterpret_cast<const uint4*>(kp + ks * 4 * EPC);
+    }
+  };
+  auto load_vs = [&](int k0) {
+#pragma unroll
+    for (int t = 0; t < NVT; ++t)
+      if (EXACT || t < nvt) vf[t] = load_v<DT>(vb + (long long)(16 * t + l15) * a.S + k0, g);
+  };
+  int k0 = kbeg + 32 * wave;
+  if (kPrefetch && k0 < klim) { load_k(k0); load_vs(k0); }
+
+  for (int i = tid; i < 16 * (CLS + EPC); i += 64 * kDecWaves) qs[i] = E(0);
+  if (owner)
+    for (int i = tid; i < CLS; i += 64 * kDecWaves) { kcur[i] = E(0); vcur[i] = E(0); }
+  __syncthreads();
+  for (int r = wave; r < nr + (owner ? 1 : 0); r += kDecWaves) {
+    const bool isk = r == nr;
+    const float* src = isk ? pj + (long long)(a.H + hk) * a.dim
+                           : pj + (long long)(hk * R + r0 + r) * a.dim;
+    float x[4];
+    head_rot_norm(src, a.dim, lane, cs, a.rd2, a.qk_norm, a.eps, x);
+    E* dst = isk ? kcur : qs + r * (CLS + EPC);
+#pragma unroll
+    for (int e = 0; e < 4; ++e)
+      if (4 * lane + e < a.dim) dst[4 * lane + e] = St<DT>::st(x[e]);
+  }
+  if (owner) {
+    const float* vsrc = pj + (long long)(a.H + a.G) * a.dim + (long long)hk * a.vdim;
+    for (int d = tid; d < a.vdim; d += 64 * kDecWaves) {
+      const E v = St<DT>::st(vsrc[d]);
+      vcur[d] = v;
+      if (r0 == 0) vb[(long long)d * a.S + pos] = v;
+    }
+  }
+  __syncthreads();
+  if (owner && r0 == 0)
+    for (int d = tid; d < DP; d += 64 * kDecWaves) kb[(long long)pos * DP + d] = kcur[d];
+
+  uint4 qf[NKS];
+#pragma unroll
+  for (int ks = 0; ks < NKS; ++ks)
+    qf[ks] = (EXACT || ks < nks)
+                 ? *reinterpret_cast<const uint4*>(qs + l15 * (CLS + EPC) + (ks * 4 + g) * EPC)
+                 : make_uint4(0, 0, 0, 0);
+  cf32x4 o[NVT];
+#pragma unroll
+  for (int t = 0; t < NVT; ++t) o[t] = cf32x4{0.f, 0.f, 0.f, 0.f};
+  float m = -INFINITY, l = 0.f;
+  if (owner && wave == 0) {  // the new key starts wave 0's softmax
+    cf32x4 sc{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int ks = 0; ks < NKS; ++ks)
+      if (EXACT || ks < nks) {
+        const uint4 kk = *reinterpret_cast<const uint4*>(kcur + (ks * 4 + g) * EPC);
+        sc = mm_piece<DT>(kk, qf[ks], sc);  // every A row is the new key: sc[e] = its score
+      }
+    m = sc[0] * a.scale_log2;
+    l = g == 0 ? 1.f : 0.f;
+#pragma unroll
+    for (int t = 0; t < NVT; ++t)
+      if (EXACT || t < nvt)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) o[t][e] = St<DT>::ld(vcur[16 * t + 4 * g + e]);
+  }
+  for (; k0 < klim; k0 += 32 * kDecWaves) {
+    if constexpr (!kPrefetch) { load_k(k0); load_vs(k0); }
+    cf32x4 s[2];
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+      s[u] = cf32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int ks = 0; ks < NKS; ++ks)
+        if (EXACT || ks < nks) s[u] = mm_piece<DT>(kf[u][ks], qf[ks], s[u]);
+    }
+    const int kn = k0 + 32 * kDecWaves;
+    if constexpr (kPrefetch) { if (kn < klim) load_k(kn); }
+    float mx = -INFINITY;
+#pragma unroll
+    for (int u = 0; u < 2; ++u)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const bool ok = k0 + 16 * u + 4 * g + e < klim;
+        s[u][e] = ok ? s[u][e] * a.scale_log2 : -INFINITY;
+        mx = fmaxf(mx, s[u][e]);
+      }
+    mx = group_max(mx);
+    const float mn = fmaxf(m, mx);  // finite: the block's first key is below klim
+    const float alpha = __builtin_amdgcn_exp2f(m - mn);
+    float rs = 0.f;
+#pragma unroll
+    for (int u = 0; u < 2; ++u)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        s[u][e] = __builtin_amdgcn_exp2f(s[u][e] - mn);
+        rs += s[u][e];
+      }
+    m = mn;
+    l = l * alpha + rs;
+    const PFrag<DT> pf = pack_p<DT>(s[0], s[1]);
+#pragma unroll
+    for (int t = 0; t < NVT; ++t)
+      if (EXACT || t < nvt) {
+        o[t] *= alpha;
+        o[t] = mm_pv<DT>(vf[t], pf, o[t]);
+      }
+    if constexpr (kPrefetch) { if (kn < klim) load_vs(kn); }
+  }
+
+  // merge of the waves
+  l = group_sum(l);
+  if (g == 0) { red_m[wave][l15] = m; red_l[wave][l15] = l; }
+#pragma unroll
+  for (int t = 0; t < NVT; ++t)
+    if (EXACT || t < nvt)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) red_o[wave][l15][16 * t + 4 * g + e] = o[t][e];
+  __syncthreads();
+  const int ngt = gridDim.x;
+  const long long pstride = 16ll * (DVP + 2);
+  float* part = a.part + ((long long)b * ngt + gt) * a.nsplit * pstride;
+  auto finish = [&](int r, int d, float num, float den) {
+    float y = num / den;
+    const int hh = hk * R + r0 + r;
+    if (a.gated)
+      y *= sigmoid32(pj[(long long)(a.H + a.G) * a.dim + (long long)a.G * a.vdim +
+                        (long long)hh * a.vdim + d]);
+    reinterpret_cast<E*>(a.out)[(long long)b * a.ldo + (long long)hh * a.vdim + d] = St<DT>::st(y);
+  };
+  for (int i = tid; i < nr * a.vdim; i += 64 * kDecWaves) {
+    const int r = i / a.vdim, d = i - r * a.vdim;
+    float M = red_m[0][r];
+#pragma unroll
+    for (int w = 1; w < kDecWaves; ++w) M = fmaxf(M, red_m[w][r]);
+    if (nact == 1 && a.sink) M = fmaxf(M, 0.f);
+    float num = 0.f, den = nact == 1 && a.sink ? __builtin_amdgcn_exp2f(-M) : 0.f;
+#pragma unroll
+    for (int w = 0; w < kDecWaves; ++w) {
+      const float f = __builtin_amdgcn_exp2f(red_m[w][r] - M);
+      num = fmaf(f, red_o[w][r][d], num);
+      den = fmaf(f, red_l[w][r], den);
+    }
+    if (nact == 1) {
+      finish(r, d, num, den);
+    } else {
+      float* pr = part + sp * pstride + (long long)r * (DVP + 2);
+      // agent-scope stores: the merging workgroup may run on another XCD
+      __hip_atomic_store(pr + 2 + d, num, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+      if (d == 0) {
+        __hip_atomic_store(pr, M, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+        __hip_atomic_store(pr + 1, den, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+      }
+    }
+  }
+  if (nact == 1) return;
+  // the last split to arrive merges all of them
+  __threadfence();
+  __syncthreads();
+  if (tid == 0) {
+    unsigned int* tk = a.ticket + (long long)b * ngt + gt;
+    const unsigned int old =
+        __hip_atomic_fetch_add(tk, 1u, __ATOMIC_ACQ_REL, __HIP_MEMORY_SCOPE_AGENT);
+    s_last = old == (unsigned int)(nact - 1);
+    if (s_last) __hip_atomic_store(tk, 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+  }
+  __syncthreads();
+  if (!s_last) return;
+  __threadfence();
+  for (int i = tid; i < nr * a.vdim; i += 64 * kDecWaves) {
+    const int r = i / a.vdim, d = i - r * a.vdim;
+    const float* pr = part + (long long)r * (DVP + 2);
+    float M = a.sink ? 0.f : -INFINITY;
+    for (int s = 0; s < nact; ++s)
+      M = fmaxf(M, __hip_atomic_load(pr + s * pstride, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT));
+    float num = 0.f, den = a.sink ? __builtin_amdgcn_exp2f(-M) : 0.f;
+    for (int s = 0; s < nact; ++s) {
+      const float* ps = pr + s * pstride;
+      const float f = __builtin_amdgcn_exp2f(
+          __hip_atomic_load(ps, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) - M);
+      num = fmaf(f, __hip_atomic_load(ps + 2 + d, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT), num);
+      den = fmaf(f, __hip_atomic_load(ps + 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT), den);
+    }
+    finish(r, d, num, den);
+  }
+}
+
+}  // namespace cake
+
+using namespace cake;
+
+static bool mix_shape_ok(int H, int G, int dim, int vdim, int DP, int DVP, int S, int rd2) {
+  return H > 0 && G > 0 && H % G == 0 && dim > 0 && vdim > 0 && DP >= dim && DP % 32 == 0 &&
+         DP <= 256 && DVP >= vdim && DVP % 16 == 0 && DVP <= 256 && S > 0 && S % 64 == 0 &&
+         rd2 >= 0 && 2 * rd2 <= dim;
+}
+
+CAKE_API int cake_mixer_prep(int dt, const void* proj, long long ldp, int N, int H, int G, int dim,
+                             int vdim, int DP, int DVP, int S, int rd2, int qk_norm, float eps,
+                             const void* cs, const int* row_pos, const int* row_slot, void* qn,
+                             void* kc, void* vc, long long k_slot, long long v_slot,
+                             hipStream_t st) {
+  if (!mix_shape_ok(H, G, dim, vdim, DP, DVP, S, rd2) || N < 0) return (int)hipErrorInvalidValue;
+  if (N == 0) return 0;
+  PrepArgs a{proj, ldp, N, H, G, dim, vdim, DP, DVP, S, rd2, qk_norm, eps, (const float2*)cs,
+             row_pos, row_slot, qn, kc, vc, k_slot, v_slot};
+  int lph = 8;
+  while (4 * lph < DP) lph <<= 1;  // <= 64
+  const long long items = (long long)N * (H + G);
+  const dim3 g1((unsigned)((items + 256 / lph - 1) / (256 / lph)));
+  const dim3 g2((N + 63) / 64, (G * ((vdim + 7) / 8) + 3) / 4);
+  CAKE_MIX_DT(dt, hipLaunchKernelGGL((mixer_prep_qk_kernel<DT>), g1, dim3(256), 0, st, a, lph);
+              hipLaunchKernelGGL((mixer_prep_v_kernel<DT>), g2, dim3(256), 0, st, a));
+  return (int)hipGetLastError();
+}
+
+template <int DT, int CLS, bool EXACT>
+static int launch_mix_flash(const MixFlashArgs& a, dim3 grid, hipStream_t st) {
+  constexpr int EPC = St<DT>::EPC, BN = DT == kF32 ? 32 : 64, NBUF = CLS <= 128 ? 2 : 1;
+  const size_t lds = (size_t)NBUF * (BN * (a.DP + EPC) + (size_t)a.DVP * (BN + EPC)) *
+                     sizeof(typename St<DT>::E);
+  static bool raised = false;
+  if (!raised) {
+    if (hipFuncSetAttribute((const void*)mixer_flash_kernel<DT, CLS, EXACT>,
+                            hipFuncAttributeMaxDynamicSharedMemorySize, 96 * 1024) != hipSuccess)
+      return (int)hipErrorInvalidValue;
+    raised = true;
+  }
+  hipLaunchKernelGGL((mixer_flash_kernel<DT, CLS, EXACT>), grid, dim3(256), lds, st, a);
+  return (int)hipGetLastError();
+}
+
+#define CAKE_MIX_CLS(FN, ...)                                                            \
+  do {                                                                                   \
+    const int cls = DP > DVP ? DP : DVP;                                                 \
+    if (cls <= 64) return DP == 64 && DVP == 64 ? FN<DT, 64, true>(__VA_ARGS__)          \
+                                                : FN<DT, 64, false>(__VA_ARGS__);        \
+    if (cls <= 128) return DP == 128 && DVP == 128 ? FN<DT, 128, true>(__VA_ARGS__)      \
+                                                   : FN<DT, 128, false>(__VA_ARGS__);    \
+    return FN<DT, 256, false>(__VA_ARGS__);                                              \
+  } while (0)
+
+CAKE_API int cake_mixer_flash(int dt, const void* qn, const void* kc, const void* vc,
+                              long long k_slot, long long v_slot, const void* seq, int B,
+                              int max_len, const void* gate, long long ldg, void* out,
+                              long long ldo, int H, int G, int dim, int vdim, int DP, int DVP,
+                              int S, int sink, float scale, hipStream_t st) {
+  if (!mix_shape_ok(H, G, dim, vdim, DP, DVP, S, 0) || B <= 0 || max_len <= 0)
+    return (int)hipErrorInvalidValue;
+  MixFlashArgs a{qn, kc, vc, k_slot, v_slot, (const SeqRow*)seq, gate, ldg, out, ldo,
+                 H, G, DP, DVP, vdim, S, sink, scale * 1.4426950408889634f};
+  const dim3 grid((max_len + 127) / 128, H, B);
+  CAKE_MIX_DT(dt, CAKE_MIX_CLS(launch_mix_flash, a, grid, st));
+  return (int)hipErrorInvalidValue;
+}
+
+template <int DT, int CLS, bool EXACT>
+static int launch_mix_dec(const MixDecArgs& a, dim3 grid, hipStream_t st) {
+  hipLaunchKernelGGL((mixer_attn_decode_kernel<DT, CLS, EXACT>), grid, dim3(64 * kDecWaves), 0, st,
+                     a);
+  return (int)hipGetLastError();
+}
+
+// f32 elements of `part` / u32 elements of `ticket` (zeroed once) for a launch
+CAKE_API long long cake_mixer_attn_part(int B, int H, int G, int DVP, int nsplit) {
+  const long long ngt = (long long)G * ((H / G + 15) / 16);
+  return (long long)B * ngt * nsplit * 16 * (DVP + 2);
+}
+
+CAKE_API int cake_mixer_attn_decode(int dt, const float* proj, long long ldp, int B, const int* pos,
+                                    const int* slot, const void* cs, int rd2, int qk_norm,
+                                    int sink, int gated, float eps, float scale, void* kc, void* vc,
+                                    long long k_slot, long long v_slot, void* out, long long ldo,
+                                    int H, int G, int dim, int vdim, int DP, int DVP, int S,
+                                    int nsplit, float* part, unsigned int* ticket, hipStream_t st) {
+  if (!mix_shape_ok(H, G, dim, vdim, DP, DVP, S, rd2) || B <= 0 || nsplit < 1 || nsplit > 64)
+    return (int)hipErrorInvalidValue;
+  MixDecArgs a{proj, ldp, pos, slot, (const float2*)cs, rd2, qk_norm, sink, gated, eps,
+               scale * 1.4426950408889634f, kc, vc, k_slot, v_slot, out, ldo, H, G, dim, vdim,
+               DP, DVP, S, nsplit, part, ticket};
+  const dim3 grid(G * ((H / G + 15) / 16), nsplit, B);
+  CAKE_MIX_DT(dt, CAKE_MIX_CLS(launch_mix_dec, a, grid, st));
+  return (int)hipErrorInvalidValue;
+}

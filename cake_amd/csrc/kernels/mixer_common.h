@@ -1,0 +1,136 @@
+// Shared pieces of the hybrid designs' layer kernels (mixer_*.hip).
+//
+// Every kernel here is a template on the storage type DT (bf16, f16 or f32).  The matrix
+// work runs on MFMA in all three: 16x16x32 for the 16-bit types, 16x16x4 f32 (true 32-bit
+// products) for f32.  Both produce the same accumulator layout — lane (l15 = l & 15,
+// g = l >> 4) holds D[4 g + e][l15] — and both take their operands as 16-byte pieces of
+// k-contiguous rows, so one source serves them: a 16-byte piece is 8 k values of one MFMA
+// (16-bit) or one k value of each of four MFMAs (f32; the k order only has to be the same
+// in both operands).
+#pragma once
+#include "common.h"
+
+namespace cake {
+
+template <int DT> struct St {  // storage element
+  using E = uint16_t;
+  static constexpr int EPC = 8;     // elements per 16-byte piece
+  static constexpr int KSTEP = 32;  // k values per qk step (4 pieces, one per lane group)
+  static __device__ __forceinline__ float ld(E v) { return to_f32<DT>(v); }
+  static __device__ __forceinline__ E st(float v) { return from_f32<DT>(v); }
+};
+template <> struct St<kF32> {
+  using E = float;
+  static constexpr int EPC = 4;
+  static constexpr int KSTEP = 16;
+  static __device__ __forceinline__ float ld(E v) { return v; }
+  static __device__ __forceinline__ E st(float v) { return v; }
+};
+
+// acc[4g + e][l15] += sum over the step's k of A[l15][k] B[l15][k] (pieces of rows)
+template <int DT>
+__device__ __forceinline__ cf32x4 mm_piece(const uint4 a, const uint4 b, cf32x4 c) {
+  if constexpr (DT == kF32) {
+    const float av[4] = {__uint_as_float(a.x), __uint_as_float(a.y), __uint_as_float(a.z),
+                         __uint_as_float(a.w)};
+    const float bv[4] = {__uint_as_float(b.x), __uint_as_float(b.y), __uint_as_float(b.z),
+                         __uint_as_float(b.w)};
+#pragma unroll
+    for (int t = 0; t < 4; ++t)
+      c = __builtin_amdgcn_mfma_f32_16x16x4f32(av[t], bv[t], c, 0, 0, 0);
+    return c;
+  } else {
+    return cmfma<DT>(a, b, c);
+  }
+}
+
+// The probabilities of two 16-key blocks (accumulator layout: key 16 blk + 4 g + e) as the
+// B operand of the value product; the A operand is V^T[d][keys 4g..4g+3] of each block.
+template <int DT> struct PFrag { uint4 p; };
+template <> struct PFrag<kF32> { float p[8]; };
+
+template <int DT>
+__device__ __forceinline__ PFrag<DT> pack_p(const cf32x4 p0, const cf32x4 p1) {
+  PFrag<DT> f;
+  if constexpr (DT == kF32) {
+#pragma unroll
+    for (int e = 0; e < 4; ++e) { f.p[e] = p0[e]; f.p[4 + e] = p1[e]; }
+  } else {
+    const auto pk = [](float lo, float hi) {
+      return (uint32_t)from_f32<DT>(lo) | ((uint32_t)from_f32<DT>(hi) << 16);
+    };
+    f.p = make_uint4(pk(p0[0], p0[1]), pk(p0[2], p0[3]), pk(p1[0], p1[1]), pk(p1[2], p1[3]));
+  }
+  return f;
+}
+
+// V^T pieces of one 16-row d tile for a 32-key pair: four keys of each block per lane group
+template <int DT> struct VFrag { uint2 lo, hi; };
+template <> struct VFrag<kF32> { float4 lo, hi; };
+
+template <int DT>
+__device__ __forceinline__ VFrag<DT> load_v(const typename St<DT>::E* row, int g) {
+  VFrag<DT> f;
+  if constexpr (DT == kF32) {
+    f.lo = *reinterpret_cast<const float4*>(row + 4 * g);
+    f.hi = *reinterpret_cast<const float4*>(row + 16 + 4 * g);
+  } else {
+    f.lo = *reinterpret_cast<const uint2*>(row + 4 * g);
+    f.hi = *reinterpret_cast<const uint2*>(row + 16 + 4 * g);
+  }
+  return f;
+}
+
+template <int DT>
+__device__ __forceinline__ cf32x4 mm_pv(const VFrag<DT>& v, const PFrag<DT>& p, cf32x4 c) {
+  if constexpr (DT == kF32) {
+    const float av[8] = {v.lo.x, v.lo.y, v.lo.z, v.lo.w, v.hi.x, v.hi.y, v.hi.z, v.hi.w};
+#pragma unroll
+    for (int t = 0; t < 8; ++t)
+      c = __builtin_amdgcn_mfma_f32_16x16x4f32(av[t], p.p[t], c, 0, 0, 0);
+    return c;
+  } else {
+    return cmfma<DT>(make_uint4(v.lo.x, v.lo.y, v.hi.x, v.hi.y), p.p, c);
+  }
+}
+
+// max / sum over the four lane groups of a 16-lane column (lanes l, l^16, l^32, l^48)
+__device__ __forceinline__ float group_max(float v) {
+  const int b = __builtin_bit_cast(int, v);
+  const auto p = __builtin_amdgcn_permlane16_swap(b, b, false, false);
+  v = fmaxf(__builtin_bit_cast(float, (int)p[0]), __builtin_bit_cast(float, (int)p[1]));
+  const int c = __builtin_bit_cast(int, v);
+  const auto q = __builtin_amdgcn_permlane32_swap(c, c, false, false);
+  return fmaxf(__builtin_bit_cast(float, (int)q[0]), __builtin_bit_cast(float, (int)q[1]));
+}
+__device__ __forceinline__ float group_sum(float v) { return xor_add<32>(xor_add<16>(v)); }
+
+// sum over a 16-lane row, every lane of the row ends with the same bits
+__device__ __forceinline__ float row16_sum(float v) {
+  v += dpp_f<kDppXor1>(v);
+  v += dpp_f<kDppXor2>(v);
+  v += dpp_f<kDppHalfMirror>(v);
+  v += dpp_f<kDppMirror>(v);
+  return v;
+}
+
+// 32-bit gates and activations (the reciprocal is IEEE division, the exponential expf)
+__device__ __forceinline__ float sigmoid32(float x) { return 1.f / (1.f + expf(-x)); }
+__device__ __forceinline__ float silu32(float x) { return x / (1.f + expf(-x)); }
+__device__ __forceinline__ float softplus32(float x) { return x > 20.f ? x : log1pf(expf(x)); }
+__device__ __forceinline__ float gelu_erf32(float x) {
+  return 0.5f * x * (1.f + erff(x * 0.70710678118654752f));
+}
+
+// One sequence of a step: its packed rows [row0, row0 + len) at positions pos0..
+struct SeqRow { int row0, len, pos0, slot; };
+
+#define CAKE_MIX_DT(dt, ...)                                          \
+  do {                                                                \
+    if ((dt) == kBF16) { constexpr int DT = kBF16; __VA_ARGS__; }     \
+    else if ((dt) == kF16) { constexpr int DT = kF16; __VA_ARGS__; }  \
+    else if ((dt) == kF32) { constexpr int DT = kF32; __VA_ARGS__; }  \
+    else return (int)hipErrorInvalidValue;                            \
+  } while (0)
+
+}  // namespace cake

@@ -1,0 +1,130 @@
+// Row kernels of the hybrid designs: embedding rows, RMS norm with an offset weight, and the
+// input of a looped pass.  Residual rows are f32 [N][ldx], ldx = width padded to 8, zeros past
+// the width; the activations they produce are [N][ldo] in the storage type, zero-padded.
+#include "mixer_common.h"
+
+namespace cake {
+
+template <int DT>
+__global__ __launch_bounds__(256) void mixer_embed_kernel(const void* table, const int* tok, int ld,
+                                                          float* x, float* x0) {
+  using E = typename St<DT>::E;
+  const E* row = reinterpret_cast<const E*>(table) + (long long)tok[blockIdx.x] * ld;
+  const long long o = (long long)blockIdx.x * ld;
+  for (int i = threadIdx.x; i < ld; i += 256) {
+    const float v = St<DT>::ld(row[i]);
+    x[o + i] = v;
+    if (x0) x0[o + i] = v;
+  }
+}
+
+// out[r] = x[rows ? rows[r] : r] * rsqrt(mean(x^2) + eps) * (off + w)
+template <int DT>
+__global__ __launch_bounds__(256) void mixer_norm_kernel(const float* x, int ldx, const int* rows,
+                                                         const float* w, float off, float eps,
+                                                         int W, void* out, int ldo) {
+  using E = typename St<DT>::E;
+  __shared__ float red[16];
+  const long long r = blockIdx.x;
+  const float* xr = x + (long long)(rows ? rows[r] : r) * ldx;
+  float4 v[8];  // rows up to 8192 stay in registers (ldx % 8 == 0, zeros past W)
+  float ss = 0.f;
+#pragma unroll
+  for (int j = 0; j < 8; ++j) {
+    const int i = (j * 256 + threadIdx.x) * 4;
+    if (i < ldx) {
+      v[j] = *reinterpret_cast<const float4*>(xr + i);
+      ss += v[j].x * v[j].x + v[j].y * v[j].y + v[j].z * v[j].z + v[j].w * v[j].w;
+    }
+  }
+  for (int i = 8192 + threadIdx.x; i < ldx; i += 256) ss += xr[i] * xr[i];
+  const float f = 1.f / sqrtf(block_sum(ss, red) / (float)W + eps);
+  E* o = reinterpret_cast<E*>(out) + r * ldo;
+#pragma unroll
+  for (int j = 0; j < 8; ++j) {
+    const int i = (j * 256 + threadIdx.x) * 4;
+    if (i < ldo) {
+      const float4 wv = *reinterpret_cast<const float4*>(w + i);
+      const float y[4] = {v[j].x * f * (off + wv.x), v[j].y * f * (off + wv.y),
+                          v[j].z * f * (off + wv.z), v[j].w * f * (off + wv.w)};
+      if constexpr (DT == kF32) {
+        *reinterpret_cast<float4*>(o + i) = make_float4(y[0], y[1], y[2], y[3]);
+      } else {
+        *reinterpret_cast<uint2*>(o + i) = make_uint2(
+            (uint32_t)St<DT>::st(y[0]) | ((uint32_t)St<DT>::st(y[1]) << 16),
+            (uint32_t)St<DT>::st(y[2]) | ((uint32_t)St<DT>::st(y[3]) << 16));
+      }
+    }
+  }
+  for (int i = 8192 + threadIdx.x; i < ldo; i += 256) o[i] = St<DT>::st(xr[i] * f * (off + w[i]));
+}
+
+// a[n] = [x[n] | x0[n] | 0] (storage type), y[n] = step (zeros past W)
+template <int DT>
+__global__ __launch_bounds__(256) void mixer_loop_rows_kernel(const float* x, const float* x0,
+                                                              int ldx, const float* step, int W,
+                                                              void* a, int lda, float* y) {
+  using E = typename St<DT>::E;
+  const long long n = blockIdx.x;
+  E* o = reinterpret_cast<E*>(a) + n * lda;
+  for (int i = threadIdx.x; i < lda; i += 256)
+    o[i] = St<DT>::st(i < W ? x[n * ldx + i] : i < 2 * W ? x0[n * ldx + i - W] : 0.f);
+  for (int i = threadIdx.x; i < ldx; i += 256) y[n * ldx + i] = i < W ? step[i] : 0.f;
+}
+
+// out[n][c] = gelu(in[n][c]) (erf), f32 storage path of the up projection
+__global__ __launch_bounds__(256) void mixer_gelu_kernel(const float* in, long long ldi, int N,
+                                                         int F, float* out, long long ldo) {
+  const long long total = (long long)N * F;
+  for (long long i = (long long)blockIdx.x * 256 + threadIdx.x; i < total;
+       i += (long long)gridDim.x * 256) {
+    const long long n = i / F;
+    const int c = (int)(i - n * F);
+    out[n * ldo + c] = gelu_erf32(in[n * ldi + c]);
+  }
+}
+
+}  // namespace cake
+
+using namespace cake;
+
+CAKE_API int cake_mixer_embed(int dt, const void* table, const int* tok, int N, int ld, float* x,
+                              float* x0, hipStream_t st) {
+  if (N < 0 || ld <= 0) return (int)hipErrorInvalidValue;
+  if (N == 0) return 0;
+  CAKE_MIX_DT(dt, hipLaunchKernelGGL((mixer_embed_kernel<DT>), dim3(N), dim3(256), 0, st, table,
+                                     tok, ld, x, x0));
+  return (int)hipGetLastError();
+}
+
+CAKE_API int cake_mixer_norm(int dt, const float* x, int ldx, const int* rows, const float* w,
+                             float off, float eps, int N, int W, void* out, int ldo,
+                             hipStream_t st) {
+  // w holds ldo f32 values (zeros past W)
+  if (N < 0 || W <= 0 || ldx % 8 || ldo != ldx || W > ldx) return (int)hipErrorInvalidValue;
+  if (N == 0) return 0;
+  CAKE_MIX_DT(dt, hipLaunchKernelGGL((mixer_norm_kernel<DT>), dim3(N), dim3(256), 0, st, x, ldx,
+                                     rows, w, off, eps, W, out, ldo));
+  return (int)hipGetLastError();
+}
+
+CAKE_API int cake_mixer_loop_rows(int dt, const float* x, const float* x0, int ldx,
+                                  const float* step, int N, int W, void* a, int lda, float* y,
+                                  hipStream_t st) {
+  if (N < 0 || W <= 0 || W > ldx || lda < 2 * W) return (int)hipErrorInvalidValue;
+  if (N == 0) return 0;
+  CAKE_MIX_DT(dt, hipLaunchKernelGGL((mixer_loop_rows_kernel<DT>), dim3(N), dim3(256), 0, st, x,
+                                     x0, ldx, step, W, a, lda, y));
+  return (int)hipGetLastError();
+}
+
+CAKE_API int cake_mixer_gelu(const float* in, long long ldi, int N, int F, float* out,
+                             long long ldo, hipStream_t st) {
+  if (N < 0 || F <= 0 || ldi < F || ldo < F) return (int)hipErrorInvalidValue;
+  if (N == 0) return 0;
+  long long g = ((long long)N * F + 255) / 256;
+  if (g > 8192) g = 8192;
+  hipLaunchKernelGGL(mixer_gelu_kernel, dim3((unsigned)g), dim3(256), 0, st, in, ldi, N, F, out,
+                     ldo);
+  return (int)hipGetLastError();
+}

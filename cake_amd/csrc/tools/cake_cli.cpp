@@ -164,6 +164,28 @@ struct EngineApi {
   void (*close)(void*);
 };
 
+cake::Json read_config(const std::string& model_dir) {
+  std::FILE* f = std::fopen((model_dir + "/config.json").c_str(), "rb");
+  if (!f) throw std::runtime_error("cannot read " + model_dir + "/config.json");
+  std::string txt;
+  char buf[4096];
+  size_t n;
+  while ((n = std::fread(buf, 1, sizeof(buf), f)) > 0) txt.append(buf, n);
+  std::fclose(f);
+  return cake::Json::parse(txt);
+}
+
+// The native engine runs the Llama family; a config.json that names another design
+// ("architecture") is served by the embedded runtime (models/registry.py).  An unreadable
+// one is left to the engine, which reports it.
+bool llama_family(const std::string& model_dir) {
+  try {
+    return !read_config(model_dir).has("architecture");
+  } catch (const std::exception&) {
+    return true;
+  }
+}
+
 bool native_text_eligible(cake::PyArgs& o, bool text, bool worker, bool has_topology) {
   const char* env = std::getenv("CAKE_NATIVE");
   if (env && std::string(env) == "0") return false;
@@ -232,14 +254,7 @@ std::vector<int32_t> owners_of(const cake::Topology* topo, int world, int num_la
 }
 
 int num_hidden_layers(const std::string& model_dir) {
-  std::FILE* f = std::fopen((model_dir + "/config.json").c_str(), "rb");
-  if (!f) throw std::runtime_error("cannot read " + model_dir + "/config.json");
-  std::string txt;
-  char buf[4096];
-  size_t n;
-  while ((n = std::fread(buf, 1, sizeof(buf), f)) > 0) txt.append(buf, n);
-  std::fclose(f);
-  return (int)cake::Json::parse(txt).get("num_hidden_layers").as_int();
+  return (int)read_config(model_dir).get("num_hidden_layers").as_int();
 }
 
 int run_native_text(cake::PyArgs& o, const cake::Topology* topo) {
@@ -523,9 +538,10 @@ int main(int argc, char** argv) {
                  topo_path.c_str());
     return 2;
   }
-  if (native_text_eligible(opts, text, worker, has_topology))
+  const bool llama = !text || llama_family(opts["model"].value);
+  if (llama && native_text_eligible(opts, text, worker, has_topology))
     return run_native_text(opts, topology.get());
-  if (native_worker_eligible(opts, text, worker)) return run_native_worker(opts, worker_node);
+  if (llama && native_worker_eligible(opts, text, worker)) return run_native_worker(opts, worker_node);
   if (native_sd_worker_eligible(opts, text, worker, worker_node))
     return run_native_sd_worker(opts, worker_node);
   return cake::run_embedded(opts);

@@ -22,6 +22,15 @@ class Token:
         return self.text or ""
 
 
+@dataclass
+class StepEntry:
+    """One sequence's share of a step: its next tokens and the places among them whose
+    logits are asked for."""
+    seq: int
+    tokens: list[int]
+    want: list[int]
+
+
 class Generator(ABC):
     MODEL_NAME: str = ""
 

@@ -1,0 +1,371 @@
+"""Hybrid decoder model: embedding -> layer runs -> final norm -> head.
+
+One step function serves prompts, decoding and mixtures of sequences (:meth:`HybridModel.step`):
+the tokens of all sequences are packed back to back, every projection is one matrix product
+over the packed rows, and only the mixers look at which row belongs to which sequence and
+position.  A layer is three stages — norm + input projections, mixer, output projections +
+residual — because its two sublayers read one norm and are summed (:mod:`.weights`).
+
+* prompt rows: MFMA GEMMs (ops/gemm.py; the feed-forward's activation and the scaled residual
+  sum in their epilogues), prompt kernels of the mixers (ops/mixers.py);
+* one token of one sequence, 16-bit: three launches per layer run (:meth:`decode_layers`, the
+  body of the captured decode graph, models/decoder.py);
+* one token of several sequences: the GEMMs over the batch, the mixers' decode kernels;
+* f32: the same kernels in their 32-bit form; the plain products are the vendor's 32-bit GEMM.
+"""
+from __future__ import annotations
+
+import contextlib
+from dataclasses import dataclass
+from functools import partial
+from pathlib import Path
+
+import torch
+
+from ...ops import gemm as G
+from ...ops import mixers as M
+from ..base import StepEntry
+from .config import AttentionMixer, HybridConfig, from_path
+from .state import StatePool
+from .weights import LayerWeights, ModelWeights
+
+# key splits of a decode-attention launch by live length: (up to this many tokens, splits)
+SPLITS = ((256, 1), (1024, 8), (4096, 16), (1 << 30, 32))
+GEN_SLOT = 0  # the generator's own sequence
+
+
+def _splits(tk: int) -> int:
+    return next(n for lim, n in SPLITS if tk <= lim)
+
+
+@dataclass
+class DecodeState:
+    """Device buffers of the captured batch-1 decode step (stable addresses)."""
+    x0: torch.Tensor       # embedding row, [Wp] f32
+    xa: torch.Tensor       # residual rows: a looped pass is entered from one into the other
+    xb: torch.Tensor
+    proj: torch.Tensor     # [max n_raw] f32
+    act: torch.Tensor      # per layer run kind: [mixer output | feed-forward] storage dtype
+    part: torch.Tensor
+    ticket: torch.Tensor
+    pos: torch.Tensor
+    seq_slot: torch.Tensor
+    tok: torch.Tensor
+    hist: torch.Tensor
+    hist_len: torch.Tensor
+    slot: torch.Tensor     # argmax key
+    thr: torch.Tensor
+    sel_ticket: torch.Tensor
+    logits: torch.Tensor
+
+
+class HybridModel:
+    backend = "hip"
+    all_local = True
+    session = 0
+
+    def __init__(self, cfg: HybridConfig, head: ModelWeights, layers: list[LayerWeights], device,
+                 dtype, max_seq: int, slots: int = 2):
+        self.cfg, self.head, self.layers = cfg, head, layers
+        self.device, self.dtype = torch.device(device), dtype
+        if self.device.type != "cuda":
+            raise ValueError("the hybrid designs run on the GPU only")
+        self.max_seq = max_seq
+        self.runs = cfg.runs()
+        self.W, self.Wp = cfg.hidden_size, cfg.width_padded
+        self.pool = StatePool(cfg, self.device, dtype, max(2, slots), max_seq)
+        self.pool.length[GEN_SLOT] = 0
+        self._rot: dict = {}
+        self._none = torch.zeros(2, device=self.device)
+        self._bufs: DecodeState | None = None
+        self._nsplit: int | None = None
+        # decode attention's split partials and arrival tickets (zeroed once, re-armed by the
+        # kernel); grown for the largest batch seen
+        self._part = self._ticket = None
+
+    # ------------------------------------------------------------------ construction
+    @classmethod
+    def load(cls, model_dir: str | Path, device, dtype, max_seq: int, slots: int = 2):
+        from ...utils.safetensors_io import ShardedCheckpoint
+        cfg = from_path(model_dir)
+        return cls.build(cfg, ShardedCheckpoint(model_dir).get, device, dtype, max_seq, slots)
+
+    @classmethod
+    def build(cls, cfg: HybridConfig, get, device, dtype, max_seq: int, slots: int = 2):
+        layers = [LayerWeights.load(get, i, cfg, device, dtype) for i in range(len(cfg.layers))]
+        return cls(cfg, ModelWeights.load(get, cfg, device, dtype), layers, device, dtype, max_seq,
+                   slots)
+
+    # ------------------------------------------------------------------ pieces
+    def _rotation(self, m: AttentionMixer) -> torch.Tensor:
+        """[S, dims] f32 (cos, sin) pairs of every cache position, computed in double."""
+        if m.rot is None or m.rot.dims < 2:
+            return self._none
+        t = self._rot.get(m.rot)
+        if t is None:
+            n = m.rot.dims // 2
+            f = float(m.rot.base) ** (-2.0 * torch.arange(n, dtype=torch.float64) / m.rot.dims)
+            a = torch.arange(self.pool.S, dtype=torch.float64)[:, None] * f
+            t = torch.stack([a.cos(), a.sin()], -1).reshape(self.pool.S, 2 * n).float()
+            t = self._rot[m.rot] = t.to(self.device).contiguous()
+        return t
+
+    def _product(self, x, w, out):
+        """out = x w^T (out: storage dtype, or f32)."""
+        if self.dtype == torch.float32:
+            torch.mm(x, w.t(), out=out) if out.is_contiguous() else out.copy_(torch.mm(x, w.t()))
+        elif out.dtype == torch.float32:
+            G.linear(x, w, epi="store32", resid=out)
+        else:
+            G.linear(x, w, out=out)
+        return out
+
+    def _product_add(self, x, w, y, alpha: float):
+        """y[:, :N] += alpha x w^T (f32)."""
+        y = y[:, :w.shape[0]]
+        if self.dtype == torch.float32:
+            y.add_(torch.mm(x, w.t()), alpha=alpha)
+        else:
+            G.linear(x, w, epi="resid32", resid=y, alpha=alpha)
+
+    def _up(self, x, w, out):
+        """out = gelu(x w^T)."""
+        if self.dtype == torch.float32:
+            M.gelu(torch.mm(x, w.t()), out)
+        else:
+            G.linear(x, w, epi="gelu", out=out)
+
+    def _split_ws(self, B: int):
+        """(partials, tickets) of decode attention for a batch of B sequences."""
+        shapes = [s for s in self.pool.shapes if isinstance(s, M.AttnShape)]
+        nsp = max(n for _, n in SPLITS)
+        need = max((s.part_floats(B, nsp) for s in shapes), default=1)
+        tick = max((B * s.tiles for s in shapes), default=1)
+        if self._part is None or self._part.numel() < need or self._ticket.numel() < tick:
+            self._part = torch.zeros(need, device=self.device, dtype=torch.float32)
+            self._ticket = torch.zeros(tick, device=self.device, dtype=torch.int32)
+        return self._part, self._ticket
+
+    # ------------------------------------------------------------------ packed rows
+    def _layer_rows(self, run, x, rows: M.Rows, nsplit: int, observe) -> None:
+        L, w = self.cfg.layers[run.layer], self.layers[run.layer]
+        m, N, cfg = L.mixer, rows.N, self.cfg
+        decode = rows.max_len == 1
+        h = torch.empty((N, self.Wp), device=self.device, dtype=self.dtype)
+        M.norm(x, w.norm32, cfg.norm_offset, cfg.eps, self.W, h)
+        new = torch.empty if w.mix_cols == w.shape.out_cols and w.ff % 8 == 0 else torch.zeros
+        mix = new((N, w.out_cols), device=self.device, dtype=self.dtype)
+        if w.ff:
+            self._up(h, w.w_in[w.n_raw:], mix[:, w.mix_cols:w.mix_cols + w.ff])
+        # the mixers' decode kernels read f32 projections, as the fused step leaves them
+        pdt = torch.float32 if decode else self.dtype
+        ncol = w.n_raw if decode else w.n_main
+        proj = torch.empty((N, M.pad_to(ncol, 8)), device=self.device, dtype=pdt)
+        self._product(h, w.w_in[:ncol], proj[:, :ncol])
+        a, b = self.pool.bufs[run.index]
+        if isinstance(m, AttentionMixer):
+            cs = self._rotation(m)
+            if decode:
+                part, ticket = self._split_ws(rows.B)
+                M.attn_decode(w.shape, proj, rows.pos, rows.slot, cs, m.qk_norm, m.sink, m.gated,
+                              cfg.eps, m.scale, a, b, mix, nsplit, part, ticket)
+            else:
+                qn = torch.empty((N, m.heads, w.shape.DP), device=self.device, dtype=self.dtype)
+                M.attn_prep(w.shape, proj, rows, cs, m.qk_norm, cfg.eps, qn, a, b)
+                gate = proj[:, w.shape.qkv_cols:w.n_main] if m.gated else None
+                M.attn_prompt(w.shape, qn, a, b, rows, gate, mix, m.scale, m.sink)
+        elif decode:
+            M.delta_decode(w.shape, proj, proj[:, w.n_main:w.n_raw], rows.pos, rows.slot, cfg.eps,
+                           **w.consts, state=a, ring=b, out=mix)
+        else:
+            ab = torch.empty((N, w.n_ab), device=self.device, dtype=torch.float32)
+            self._product(h, w.w_in[w.n_main:w.n_raw], ab)
+            M.delta_prompt(w.shape, proj, ab, rows, cfg.eps, **w.consts, state=a, ring=b, out=mix)
+        self._product_add(mix, w.w_out, x, cfg.residual_mult)
+        if observe is not None:
+            observe(x[:, :self.W])
+
+    def _forward_rows(self, rows: M.Rows, observe=None) -> torch.Tensor:
+        """Residual rows [N, Wp] f32 after every layer run."""
+        N, head = rows.N, self.head
+        x = torch.empty((N, self.Wp), device=self.device, dtype=torch.float32)
+        x0 = torch.empty_like(x) if self.cfg.loop is not None else None
+        M.embed(head.embed, rows.tok, x, x0)
+        nsplit = _splits(max(p0 + n for _, n, p0, _ in rows.host))
+        for run in self.runs:
+            if run.enter is not None:
+                pair = torch.empty((N, head.loop_in.shape[1]), device=self.device,
+                                   dtype=self.dtype)
+                y = torch.empty_like(x)
+                M.loop_rows(x, x0, head.loop_step[run.enter], self.W, pair, y)
+                self._product_add(pair, head.loop_in, y, 1.0)
+                x = y
+            self._layer_rows(run, x, rows, nsplit, observe)
+        return x
+
+    def _logits(self, x, take: list[int]) -> torch.Tensor:
+        """Logits [len(take), V] f32 of the given residual rows."""
+        V = self.cfg.vocab_size
+        out = torch.empty((len(take), V), device=self.device, dtype=torch.float32)
+        if take:
+            sel = torch.tensor(take, dtype=torch.int32).to(self.device)
+            h = torch.empty((len(take), self.Wp), device=self.device, dtype=self.dtype)
+            M.norm(x, self.head.norm32, self.cfg.norm_offset, self.cfg.eps, self.W, h, rows=sel)
+            self._product(h, self.head.lm_head, out)
+        return out
+
+    # ------------------------------------------------------------------ steps
+    def open_sequence(self) -> int:
+        return self.pool.open()
+
+    def close_sequence(self, sid: int) -> None:
+        self.pool.close(sid)
+
+    @torch.no_grad()
+    def step(self, entries: list[StepEntry], observe=None) -> list[torch.Tensor]:
+        """Feed each sequence its next tokens as one batch; logits [len(want), V] per entry.
+        ``observe`` is called with the packed residual rows after every layer run."""
+        if len({e.seq for e in entries}) != len(entries):
+            raise ValueError("a sequence appears twice in one step")
+        V = self.cfg.vocab_size
+        for e in entries:
+            if not e.tokens or not all(0 <= t < V for t in e.tokens) or \
+                    not all(0 <= w < len(e.tokens) for w in e.want):
+                raise ValueError("step: tokens or wanted places out of range")
+            if self.pool.length[e.seq] + len(e.tokens) > self.max_seq:
+                raise ValueError(f"sequence {e.seq} exceeds max_seq {self.max_seq}")
+        seqs = [(e.seq, self.pool.reserve(e.seq, len(e.tokens)), e.tokens) for e in entries]
+        if len(seqs) == 1 and len(entries[0].tokens) == 1 and self.dtype != torch.float32 \
+                and observe is None:
+            slot, pos, (tok,) = seqs[0]
+            b = self.decode_buffers()
+            b.tok.fill_(tok)
+            b.pos.fill_(pos)
+            b.seq_slot.fill_(slot)
+            self.decode_embed(b)
+            with self.decode_eager(pos):
+                x = self.decode_layers(b, range(len(self.runs)))
+            out = self._logits(x.view(1, -1), [0] * len(entries[0].want))
+            b.seq_slot.fill_(GEN_SLOT)
+            return [out]
+        rows = M.Rows.pack(seqs, self.device)
+        x = self._forward_rows(rows, observe)
+        take = [h[0] + w for h, e in zip(rows.host, entries) for w in e.want]
+        return list(self._logits(x, take).split([len(e.want) for e in entries]))
+
+    # ------------------------------------------------------------------ generator interface
+    def reset(self) -> None:
+        self.pool.length[GEN_SLOT] = 0
+
+    def forward(self, tokens: list[int], pos0: int) -> torch.Tensor:
+        """Logits (f32 [V]) of the last of `tokens`, fed at positions pos0.. of the
+        generator's sequence."""
+        self.pool.length[GEN_SLOT] = pos0
+        return self.step([StepEntry(GEN_SLOT, list(tokens), [len(tokens) - 1])])[0][0]
+
+    # ------------------------------------------------------------------ decode hooks
+    @property
+    def device_decode(self) -> bool:
+        """Tokens can run as the fused step of a captured graph (16-bit weights)."""
+        return self.dtype != torch.float32
+
+    @property
+    def decode_version(self) -> int:
+        """Changes when captured graphs no longer fit the model's buffers."""
+        return self.pool.version
+
+    @property
+    def num_decode_layers(self) -> int:
+        return len(self.runs)
+
+    def decode_buffers(self) -> DecodeState:
+        if self._bufs is None:
+            dev, f, i32 = self.device, torch.float32, torch.int32
+            z = partial(torch.zeros, device=dev)
+            part, ticket = self._split_ws(1)
+            self._bufs = DecodeState(
+                x0=z(self.Wp, dtype=f), xa=z(self.Wp, dtype=f), xb=z(self.Wp, dtype=f),
+                proj=z(max(w.n_raw for w in self.layers), dtype=f),
+                act=z((len(self.layers), max(w.out_cols for w in self.layers)), dtype=self.dtype),
+                part=part, ticket=ticket, pos=z(1, dtype=i32), seq_slot=z(1, dtype=i32),
+                tok=z(1, dtype=i32), hist=z(self.max_seq, dtype=i32), hist_len=z(1, dtype=i32),
+                slot=z(1, dtype=torch.int64), thr=z(1, dtype=i32), sel_ticket=z(1, dtype=i32),
+                logits=z(self.cfg.vocab_size, dtype=f))
+        return self._bufs
+
+    def decode_state(self, b: DecodeState) -> list[torch.Tensor]:
+        return [b.tok, b.pos, b.hist_len, b.x0, *self.pool.recurrent(GEN_SLOT)]
+
+    def decode_embed(self, b: DecodeState) -> None:
+        M.embed(self.head.embed, b.tok, b.x0)
+
+    def decode_layers(self, b: DecodeState, layers) -> torch.Tensor:
+        """Layer runs of one token at device position b.pos of slot b.seq_slot, three launches
+        each (16-bit weights; graph-capturable); returns the residual row.  The first run of
+        a step reads b.x0."""
+        cfg, x = self.cfg, b.x0
+        nsplit = self._nsplit or max(n for _, n in SPLITS)
+        for r in layers:
+            run = self.runs[r]
+            L, w = cfg.layers[run.layer], self.layers[run.layer]
+            m = L.mixer
+            if run.enter is not None:
+                y = b.xb if x is b.xa else b.xa
+                M.loop_in(x, b.x0, self.head.loop_step[run.enter], self.head.loop_in, self.W, y)
+                x = y
+            mix = b.act[run.layer, :w.out_cols]
+            M.layer_in(x, w.norm, cfg.eps, cfg.norm_offset, self.W, w.w_in, w.n_raw, b.proj,
+                       mix[w.mix_cols:])
+            ka, kb = self.pool.bufs[run.index]
+            proj = b.proj[:w.n_raw].view(1, -1)
+            if isinstance(m, AttentionMixer):
+                M.attn_decode(w.shape, proj, b.pos, b.seq_slot, self._rotation(m), m.qk_norm,
+                              m.sink, m.gated, cfg.eps, m.scale, ka, kb, mix.view(1, -1), nsplit,
+                              b.part, b.ticket)
+            else:
+                M.delta_decode(w.shape, proj, proj[:, w.n_main:], b.pos, b.seq_slot, cfg.eps,
+                               **w.consts, state=ka, ring=kb, out=mix.view(1, -1))
+            y = b.xa if x is b.x0 else x
+            M.layer_out(mix, w.w_out, cfg.residual_mult, x, y)
+            x = y
+        self._last = x
+        return x
+
+    def decode_head(self, b: DecodeState) -> None:
+        from ...ops import hip as K
+        h = self.head
+        K.norm_gemv_f32_off(self._last, h.norm, self.cfg.eps, self.cfg.norm_offset, self.W,
+                            h.lm_head, b.logits)
+
+    def decode_head_select(self, b: DecodeState, last_n: int, penalty: float) -> None:
+        from ...ops import hip as K
+        h = self.head
+        K.head_select_off(self._last, h.norm, self.cfg.eps, self.cfg.norm_offset, self.W,
+                          h.lm_head, b.logits, b.hist, b.hist_len, last_n, penalty, b.slot,
+                          b.sel_ticket, b.tok, b.pos, h.embed, b.x0)
+
+    @contextlib.contextmanager
+    def _split_scope(self, n: int):
+        prev, self._nsplit = self._nsplit, n
+        try:
+            yield
+        finally:
+            self._nsplit = prev
+
+    def decode_buckets(self) -> list:
+        top = _splits(self.max_seq)
+        return [(n, partial(self._split_scope, n)) for _, n in SPLITS if n <= top]
+
+    def decode_need(self, tk: int) -> int:
+        return _splits(tk)
+
+    def decode_eager(self, pos: int):
+        return self._split_scope(_splits(pos + 1))
+
+    def decode_check(self, b: DecodeState) -> None:
+        """Nothing to check: no launch of a step waits on another workgroup."""
+
+    def prefill_logits(self, prompt: list[int], out: torch.Tensor) -> None:
+        self.reset()
+        out.copy_(self.forward(prompt, 0))
+        self.decode_buffers().seq_slot.fill_(GEN_SLOT)

@@ -1,0 +1,71 @@
+"""Per-sequence state of a hybrid model: a pool of slots.
+
+Every layer run owns its part of every slot: attention a K and a transposed V cache of
+``max_seq`` positions, the delta rule its 32-bit state and the ring of its convolution's last
+inputs.  A slot is handed out with position 0; the kernels start a sequence at position 0 from
+zeros, so a slot that is used again needs no clearing.
+"""
+from __future__ import annotations
+
+import torch
+
+from ...ops.mixers import AttnShape, pad_to
+from .config import HybridConfig
+from .weights import mixer_shape
+
+
+class StatePool:
+    def __init__(self, cfg: HybridConfig, device, dtype, slots: int, max_seq: int):
+        self.cfg = cfg
+        self.device, self.dtype = torch.device(device), dtype
+        self.S = pad_to(max_seq, 64)
+        self.max_seq = max_seq
+        self.slots = 0
+        self.version = 0                   # counts moves of the buffers
+        self._old: list = []               # superseded buffers: captured graphs may point at them
+        self.shapes = [mixer_shape(cfg.layers[r.layer].mixer) for r in cfg.runs()]
+        self.bufs: list[tuple[torch.Tensor, torch.Tensor]] = []
+        self.length: dict[int, int] = {}   # open slot -> tokens held
+        self._grow(slots)
+
+    def _part(self, sh, n: int) -> tuple[torch.Tensor, torch.Tensor]:
+        kw = dict(device=self.device)
+        if isinstance(sh, AttnShape):
+            return (torch.zeros((n, sh.kv_heads, self.S, sh.DP), dtype=self.dtype, **kw),
+                    torch.zeros((n, sh.kv_heads, sh.DVP, self.S), dtype=self.dtype, **kw))
+        return (torch.zeros((n, sh.heads, sh.dim, sh.EP), dtype=torch.float32, **kw),
+                torch.zeros((n, sh.taps, sh.channels), dtype=torch.float32, **kw))
+
+    def _grow(self, slots: int) -> None:
+        new = [self._part(sh, slots) for sh in self.shapes]
+        for (a, b), (x, y) in zip(self.bufs, new):
+            x[:self.slots].copy_(a)
+            y[:self.slots].copy_(b)
+        if self.bufs:
+            self._old.append(self.bufs)
+            self.version += 1
+        self.bufs, self.slots = new, slots
+
+    def open(self) -> int:
+        free = next((s for s in range(self.slots) if s not in self.length), None)
+        if free is None:
+            free = self.slots
+            self._grow(2 * self.slots)
+        self.length[free] = 0
+        return free
+
+    def close(self, slot: int) -> None:
+        del self.length[slot]
+
+    def reserve(self, slot: int, n: int) -> int:
+        """Positions for n more tokens of a sequence; returns the first."""
+        p0 = self.length[slot]
+        if p0 + n > self.max_seq:
+            raise ValueError(f"sequence length {p0 + n} exceeds max_seq {self.max_seq}")
+        self.length[slot] = p0 + n
+        return p0
+
+    def recurrent(self, slot: int) -> list[torch.Tensor]:
+        """The parts of a slot that a token overwrites rather than appends to."""
+        return [t[slot] for sh, part in zip(self.shapes, self.bufs)
+                if not isinstance(sh, AttnShape) for t in part]

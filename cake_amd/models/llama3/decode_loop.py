@@ -15,7 +15,7 @@ from typing import Callable
 
 import torch
 
-from .model import DeviceDecoder
+from ..decoder import DeviceDecoder
 
 
 @dataclass
@@ -118,9 +118,7 @@ def _check(dec: DeviceDecoder) -> None:
     """Raise (and re-arm) when a decode launch of this run gave up in a bounded spin:
     the split-K attention merge's error word (tickets[2 nkv]) or a persistent-decode
     hand-off — its tokens are invalid (one host read, after the loop's final sync)."""
-    stack = getattr(dec.m, "stack", None)
-    if stack is not None and getattr(stack, "backend", "hip") == "hip":
-        stack.mk_check(dec.bufs)
+    dec.m.decode_check(dec.bufs)
 
 
 def _run_native(dec: DeviceDecoder, n_steps: int, eos_ids, on_token) -> DecodeStats:
@@ -132,7 +130,7 @@ def _run_native(dec: DeviceDecoder, n_steps: int, eos_ids, on_token) -> DecodeSt
     # the device history holds one token per position up to the current one: its
     # length is host_pos + 1 (no device read-back — a sync — inside the timed loop)
     base = dec.host_pos + 1
-    room = min(dec.bufs.hist.numel() - base, dec.m.stack.max_seq - 1 - dec.host_pos)
+    room = min(dec.bufs.hist.numel() - base, dec.m.max_seq - 1 - dec.host_pos)
     n = min(n_steps, room // k * k)
     if n <= 0:
         return st

@@ -31,7 +31,8 @@ from ..base import TextGenerator, Token
 from ..chat import History, Message
 from ..sampling import LogitsProcessor, SamplingConfig
 from ...ops import reference as R
-from .model import DeviceDecoder, LlamaModel
+from ..decoder import DeviceDecoder
+from .model import LlamaModel
 
 DEFAULT_EOS_TOKEN = "</s>"
 
@@ -124,7 +125,7 @@ class LLamaGenerator(TextGenerator):
         self.index_pos = 0
 
     def _fast_path(self) -> bool:
-        return self.model.backend == "hip" and self.model.all_local
+        return self.model.device_decode
 
     def next_token(self, index: int) -> Token:
         if self.generated == 0:
@@ -182,7 +183,7 @@ class LLamaGenerator(TextGenerator):
         if first.is_end_of_stream and stop_at_eos:
             return out
         # every further token needs a KV-cache row: clamp to the cache (max_seq)
-        max_tokens = min(max_tokens, self.model.stack.max_seq - len(self.tokens) + 1)
+        max_tokens = min(max_tokens, self.model.max_seq - len(self.tokens) + 1)
         if not self._fast_path():
             for i in range(1, max_tokens):
                 t = self.next_token(i)

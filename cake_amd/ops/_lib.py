@@ -1,6 +1,9 @@
-"""ctypes binding of ``libcake_kernels.so`` (the gfx950 HIP kernels).
+"""ctypes binding of the gfx950 HIP kernel libraries.
 
-The library exposes a plain C ABI; each entry point takes raw device pointers
+``libcake_kernels.so`` (:func:`kernels`) holds most of them; the GEMM and the
+hybrid designs' layers are libraries of their own (:func:`library`).
+
+The libraries expose a plain C ABI; each entry point takes raw device pointers
 plus the HIP stream to launch on.  We pass torch's *current* stream so that a
 ``torch.cuda.graph`` capture records our launches like any torch op.
 
@@ -14,7 +17,8 @@ import os
 import threading
 from pathlib import Path
 
-_LIB_PATH = Path(__file__).resolve().parent.parent / "lib" / "libcake_kernels.so"
+_LIB_DIR = Path(__file__).resolve().parent.parent / "lib"
+_LIB_PATH = _LIB_DIR / "libcake_kernels.so"
 _lock = threading.Lock()
 _lib = None
 
@@ -106,6 +110,32 @@ def kernels():
     return _lib
 
 
+_loaded: dict = {}
+
+
+def library(name: str):
+    """Load (once) ``libcake_<name>.so`` — "gemm" or "mixers" — with its signatures."""
+    lib = _loaded.get(name)
+    if lib is not None:
+        return lib
+    with _lock:
+        lib = _loaded.get(name)
+        if lib is None:
+            import torch  # noqa: F401  (HIP runtime must be loaded by torch first)
+
+            path = _LIB_DIR / f"libcake_{name}.so"
+            if not path.exists():
+                raise KernelError(
+                    f"{path} not built; run `python -m cake_amd.build` (hipcc gfx950)")
+            lib = C.CDLL(str(path), mode=C.RTLD_GLOBAL)
+            for fname, argtypes in _LIB_SIGS.get(name, {}).items():
+                fn = getattr(lib, fname)
+                fn.argtypes = argtypes
+                fn.restype = C.c_int
+            _loaded[name] = lib
+    return lib
+
+
 def available() -> bool:
     try:
         kernels()
@@ -153,3 +183,29 @@ _OPTIONAL = {"cake_mk_gstride", "cake_mk_grid", "cake_mk_supported", "cake_mk_de
 _SIGS["cake_mk_set_stamps"] = [P]
 _SIGS["cake_mk_set_tuning"] = [I, I, I, I]
 _SIGS["cake_attn_debug_drop_partials"] = [I]
+
+L = C.c_longlong
+_SIGS.update({
+    "cake_gemv_norm_f32_off": [I, P, P, F, F, I, P, I, I, P, P],
+    "cake_head_select_off": [I, P, P, F, F, I, P, I, I, P, P, P, I, F, P, P, P, P, I, P, P, P],
+})
+# entry points of the separate libraries (int hipError_t); the GEMM's are bound in ops/gemm.py
+_LIB_SIGS = {
+    "mixers": {
+        "cake_mixer_embed": [I, P, P, I, I, P, P, P],
+        "cake_mixer_norm": [I, P, I, P, P, F, F, I, I, P, I, P],
+        "cake_mixer_loop_rows": [I, P, P, I, P, I, I, P, I, P, P],
+        "cake_mixer_gelu": [P, L, I, I, P, L, P],
+        "cake_mixer_in": [I, P, P, F, F, I, P, I, I, I, P, P, P],
+        "cake_mixer_out": [I, P, P, I, I, F, P, P, P],
+        "cake_mixer_loop": [I, P, P, P, P, I, I, P, P],
+        "cake_mixer_prep": [I, P, L, I, I, I, I, I, I, I, I, I, I, F, P, P, P, P, P, P, L, L, P],
+        "cake_mixer_flash": [I, P, P, P, L, L, P, I, I, P, L, P, L, I, I, I, I, I, I, I, I, F, P],
+        "cake_mixer_attn_decode": [I, P, L, I, P, P, P, I, I, I, I, F, F, P, P, L, L, P, L, I, I,
+                                   I, I, I, I, I, I, P, P, P],
+        "cake_mixer_delta_prefill": [I, P, L, P, L, I, I, I, I, I, I, I, F, P, P, P, P, P, P, P,
+                                     P, P, P, P, P, L, L, P, P, P, P, I, P, L, P],
+        "cake_mixer_delta_decode": [I, P, L, P, L, I, I, I, I, I, I, I, F, P, P, P, P, P, P, L, L,
+                                    P, P, P, L, P],
+    },
+}

@@ -16,7 +16,7 @@ import ctypes as C
 
 import torch
 
-from ._lib import check, kernels
+from ._lib import check, kernels, library
 
 EPI = {"store": 0, "resid32": 1, "add16": 2, "swiglu": 3, "geglu": 4, "store32": 6, "silu": 7,
        "quick_gelu": 8, "gelu": 9}
@@ -55,18 +55,28 @@ _zeros: dict = {}
 
 
 def _lib():
+    """The GEMM library (libcake_gemm.so)."""
     global _bound
-    lib = kernels()
+    lib = library("gemm")
     if not _bound:
         P, I, L = C.c_void_p, C.c_int, C.c_longlong
-        lib.cake_gemm.argtypes = [I, I, I, I, P, L, P, L, P, L, P, P, L, P, P, I, I, I, P]
-        lib.cake_gemm.restype = I
+        lib.cake_gemm_scaled.argtypes = [I, I, I, I, P, L, P, L, P, L, P, P, L, P, P, I, I, I,
+                                         C.c_float, P]
+        lib.cake_gemm_scaled.restype = I
         lib.cake_gemm_ws_floats.argtypes = [I, I, I, I, I, I]
         lib.cake_gemm_ws_floats.restype = L
-        lib.cake_blaslt_gemm.argtypes = [I, I, P, L, P, L, P, L, I, I, I, P, C.c_size_t, P]
-        lib.cake_blaslt_gemm.restype = I
         _bound = True
     return lib
+
+
+def _lib_blaslt():
+    """The library GEMM's entry point (csrc/driver/blaslt.cpp, in libcake_kernels.so)."""
+    fn = kernels().cake_blaslt_gemm
+    if fn.argtypes is None:
+        P, I, L = C.c_void_p, C.c_int, C.c_longlong
+        fn.argtypes = [I, I, P, L, P, L, P, L, I, I, I, P, C.c_size_t, P]
+        fn.restype = I
+    return fn
 
 
 def _zeros16(dev) -> torch.Tensor:
@@ -211,18 +221,18 @@ def _rows_view(t: torch.Tensor, name: str) -> tuple[torch.Tensor, int]:
 def linear(x: torch.Tensor, w: torch.Tensor, bias: torch.Tensor | None = None, *,
            epi: str = "store", out: torch.Tensor | None = None,
            resid: torch.Tensor | None = None, cfg: int | None = None,
-           splits: int | None = None) -> torch.Tensor:
+           splits: int | None = None, alpha: float = 1.0) -> torch.Tensor:
     """y = epilogue(x @ w.T) on MFMA.
 
     x [..., K] (16-bit, unit column stride, any row stride that is a multiple of
     8); w [N, K] ([2F, K] for the gated epilogues: rows [0, F) gate/h, [F, 2F)
     up/gate).  Epilogues:
       store   -> out [..., N] = y (+ bias)
-      resid32 -> resid (f32 [..., N]) += y (+ bias); returns resid
+      resid32 -> resid (f32 [..., N]) += alpha * (y (+ bias)); returns resid
       add16   -> out = y (+ bias) + resid (16-bit [..., N])
       swiglu  -> out [..., F] = silu(y_gate) * y_up
       geglu   -> out [..., F] = (y_h + b_h) * gelu_tanh(y_gate + b_gate)
-      store32 -> resid (f32 [..., N], any row stride) = y (+ bias); returns resid
+      store32 -> resid (f32 [..., N], any row stride) = alpha * (y (+ bias)); returns resid
       silu    -> out = silu(y (+ bias))
       quick_gelu / gelu -> out = act(y (+ bias)) (CLIP MLP: x*sigmoid(1.702x) / erf GELU)
     """
@@ -287,7 +297,9 @@ def linear(x: torch.Tensor, w: torch.Tensor, bias: torch.Tensor | None = None, *
     c0, s0 = plan(M, Nv, K, epi)
     cfg = c0 if cfg is None else cfg
     lib_ok = epi != "swiglu" or (ldc == N and N % 8 == 0 and out2.data_ptr() % 16 == 0)
-    if cfg == LIB and bias is None and epi in LIB_EPIS and lib_ok:
+    if alpha != 1.0 and not f32_out:
+        raise ValueError(f"{epi} takes no alpha")
+    if cfg == LIB and bias is None and epi in LIB_EPIS and lib_ok and alpha == 1.0:
         _lib_gemm(x2, lda, w, ldb, epi, out2, ldc, r2 if f32_out else None, ldr, M, N, K)
         return resid if f32_out else out
     if cfg == LIB:  # an epilogue / bias / strided output the library form does not carry
@@ -296,11 +308,11 @@ def linear(x: torch.Tensor, w: torch.Tensor, bias: torch.Tensor | None = None, *
     # the kernel library sizes it (an in-kernel pair needs its slabs only)
     ws = _workspace(x.device, int(_lib().cake_gemm_ws_floats(
         int(cfg), int(splits), M, N, K, 1 if Nv != N else 0))) if splits > 1 else None
-    check(_lib().cake_gemm(_DT[x.dtype], EPI[epi], int(cfg), int(splits), x2.data_ptr(), lda,
-                           w.data_ptr(), ldb, cptr, ldc,
-                           None if bias is None else bias.data_ptr(), rptr, ldr,
-                           None if ws is None else ws.data_ptr(), _zeros16(x.device).data_ptr(),
-                           M, N, K, torch.cuda.current_stream().cuda_stream), "gemm")
+    check(_lib().cake_gemm_scaled(
+        _DT[x.dtype], EPI[epi], int(cfg), int(splits), x2.data_ptr(), lda, w.data_ptr(), ldb, cptr,
+        ldc, None if bias is None else bias.data_ptr(), rptr, ldr,
+        None if ws is None else ws.data_ptr(), _zeros16(x.device).data_ptr(), M, N, K,
+        float(alpha), torch.cuda.current_stream().cuda_stream), "gemm")
     return resid if f32_out else out
 
 
@@ -315,7 +327,7 @@ def _lib_gemm(x2, lda, w, ldb, epi, out2, ldc, r2, ldr, M, N, K) -> None:
     dt = _DT[x2.dtype]
 
     def run(mode, cptr, ld, n):
-        check(_lib().cake_blaslt_gemm(dt, mode, x2.data_ptr(), lda, w.data_ptr(), ldb, cptr, ld,
+        check(_lib_blaslt()(dt, mode, x2.data_ptr(), lda, w.data_ptr(), ldb, cptr, ld,
                                       M, n, K, ws.data_ptr(), _LIB_WS_BYTES, st), "blaslt gemm")
     if epi == "store":
         run(0, out2.data_ptr(), ldc, N)

@@ -1086,3 +1086,44 @@ def to_rgb8(img, nhwc: bool = False) -> torch.Tensor:
     check(kernels().cake_to_rgb8(_dt(img), _p(img), B, H, W, int(nhwc), _p(out), _stream()),
           "to_rgb8")
     return out
+
+
+# ---------------------------------------------------------------------------
+# head with a norm weight stored around an offset (hybrid designs)
+# ---------------------------------------------------------------------------
+
+def norm_gemv_f32_off(resid, norm_w, eps, off: float, width: int, w, out):
+    """out (f32) = w @ (resid / rms * (off + norm_w)), the mean over the first `width`
+    columns (zeros past them)."""
+    N, K = w.shape
+    _req(resid, "resid", dtype=torch.float32, numel=K)
+    _req(norm_w, "norm_w", dtype=w.dtype, shape=(K,))
+    _req(w, "w")
+    _req(out, "out", dtype=torch.float32, numel=N)
+    check(kernels().cake_gemv_norm_f32_off(_dt(w), _p(resid), _p(norm_w), float(eps), float(off),
+                                           int(width), _p(w), K, N, _p(out), _stream()),
+          "gemv_norm_f32_off")
+
+
+def head_select_off(resid, norm_w, eps, off: float, width: int, w, logits, hist, hist_len,
+                    last_n: int, penalty: float, slot, ticket, tok, pos, embed, emb_out) -> None:
+    """:func:`head_select` for such a norm; the next step's input row goes to emb_out."""
+    N, K = w.shape
+    _req(resid, "resid", dtype=torch.float32, numel=K)
+    _req(norm_w, "norm_w", dtype=w.dtype, shape=(K,))
+    _req(w, "w")
+    _req(logits, "logits", dtype=torch.float32, numel=N)
+    _req(slot, "slot", dtype=torch.int64, numel=1)
+    _req(ticket, "ticket", dtype=torch.int32, numel=1)
+    for t, n in ((tok, "tok"), (hist, "hist"), (hist_len, "hist_len"), (pos, "pos")):
+        _req(t, n, dtype=torch.int32)
+    if not 0 <= int(last_n) <= HEAD_SELECT_MAX_LAST_N:
+        raise ValueError(f"head_select: last_n {last_n} > {HEAD_SELECT_MAX_LAST_N}")
+    _req(embed, "embed", dtype=w.dtype)
+    _req(emb_out, "emb_out", dtype=torch.float32, numel=K)
+    if embed.dim() != 2 or embed.shape[1] != K:
+        raise ValueError(f"head_select: embed {tuple(embed.shape)} does not match H={K}")
+    check(kernels().cake_head_select_off(
+        _dt(w), _p(resid), _p(norm_w), float(eps), float(off), int(width), _p(w), K, N, _p(logits),
+        _p(hist), _p(hist_len), int(last_n), float(penalty), _p(slot), _p(ticket), _p(tok),
+        _p(pos), hist.numel(), _p(embed), _p(emb_out), _stream()), "head_select_off")

@@ -1,0 +1,353 @@
+"""Torch-tensor wrappers of the hybrid designs' layer kernels (csrc/kernels/mixer_*.hip).
+
+Storage types bf16, f16 and f32 (f32: true 32-bit products).  As in :mod:`.hip`, shapes,
+dtypes and strides are validated on the host before every launch and nothing falls back to
+PyTorch.  Prompt rows of several sequences are packed back to back; :class:`Rows` carries
+where each row belongs.
+"""
+from __future__ import annotations
+
+from dataclasses import dataclass
+
+import torch
+
+from ._lib import check, library
+
+DT = {torch.bfloat16: 0, torch.float16: 1, torch.float32: 2}
+MAX_HEAD = 256   # largest head size the kernels hold
+MAX_SPLIT = 64   # key splits of one decode-attention launch
+
+
+def _lib():
+    return library("mixers")
+
+
+def _stream() -> int:
+    return torch.cuda.current_stream().cuda_stream
+
+
+def pad_to(n: int, m: int) -> int:
+    return -(-n // m) * m
+
+
+def _vec(t, name, dtype, numel=None):
+    if not t.is_cuda or t.dtype != dtype or not t.is_contiguous():
+        raise ValueError(f"{name}: expected a contiguous {dtype} device tensor")
+    if numel is not None and t.numel() < numel:
+        raise ValueError(f"{name}: expected >= {numel} elements, got {t.numel()}")
+    return t.data_ptr()
+
+
+def _mat(t, name, dtype, rows, cols):
+    """[rows, >= cols] with unit column stride -> (pointer, row stride)."""
+    if not t.is_cuda or t.dtype != dtype or t.dim() != 2 or t.stride(1) != 1 or \
+            t.shape[0] < rows or t.shape[1] < cols or (t.shape[0] > 1 and t.stride(0) < t.shape[1]):
+        raise ValueError(f"{name}: expected a [{rows}, {cols}] {dtype} device matrix, got "
+                         f"{tuple(t.shape)} {t.dtype} strides {t.stride()}")
+    return t.data_ptr(), t.stride(0)
+
+
+@dataclass
+class Rows:
+    """Packed rows of one step: B sequences, N rows (int32 device tensors)."""
+    N: int
+    B: int
+    max_len: int
+    tok: torch.Tensor    # [N]
+    pos: torch.Tensor    # [N]
+    slot: torch.Tensor   # [N]
+    first: torch.Tensor  # [N] packed row of the sequence's first token of this step
+    seq: torch.Tensor    # [B, 4]: first row, length, first position, slot
+    host: list           # [(first row, length, first position, slot)]
+
+    @classmethod
+    def pack(cls, seqs: list[tuple[int, int, list[int]]], device) -> "Rows":
+        """seqs: (slot, first position, tokens)."""
+        tok, pos, slot, first, host = [], [], [], [], []
+        for s, p0, toks in seqs:
+            r0, n = len(tok), len(toks)
+            if n == 0:
+                raise ValueError("a sequence of a step needs at least one token")
+            host.append((r0, n, p0, s))
+            tok += list(toks)
+            pos += range(p0, p0 + n)
+            slot += [s] * n
+            first += [r0] * n
+        N, B = len(tok), len(host)
+        flat = torch.tensor(tok + pos + slot + first + [x for h in host for x in h],
+                            dtype=torch.int32).to(device)
+        t = [flat[i * N:(i + 1) * N] for i in range(4)]
+        return cls(N, B, max(h[1] for h in host), *t, flat[4 * N:].view(B, 4), host)
+
+
+def embed(table, tok, x, x0=None):
+    """x [N, ld] f32 (and x0) = table rows; table [V, ld]."""
+    N, ld = tok.numel(), table.shape[1]
+    check(_lib().cake_mixer_embed(DT[table.dtype], _vec(table, "table", table.dtype),
+                                  _vec(tok, "tok", torch.int32), N, ld,
+                                  _vec(x, "x", torch.float32, N * ld),
+                                  None if x0 is None else _vec(x0, "x0", torch.float32, N * ld),
+                                  _stream()), "mixer_embed")
+
+
+def norm(x, w, offset: float, eps: float, width: int, out, rows=None):
+    """out[r] = x[rows[r] or r] / rms * (offset + w); x [*, ld] f32, w [ld] f32, out [R, ld]."""
+    R, ld = out.shape
+    xp, ldx = _mat(x, "x", torch.float32, 1 if rows is not None else R, ld)
+    if ldx != ld or not out.is_contiguous() or ld % 8:
+        raise ValueError("norm: x and out need the same row length, a multiple of 8")
+    check(_lib().cake_mixer_norm(DT[out.dtype], xp, ld,
+                                 None if rows is None else _vec(rows, "rows", torch.int32, R),
+                                 _vec(w, "w", torch.float32, ld), float(offset), float(eps), R,
+                                 int(width), out.data_ptr(), ld, _stream()), "mixer_norm")
+
+
+def loop_rows(x, x0, step, width: int, a, y):
+    """a [N, >= 2 width] = [x | x0 | 0] in the storage type, y [N, ld] f32 = step."""
+    N, ld = x.shape
+    ap, lda = _mat(a, "a", a.dtype, N, 2 * width)
+    check(_lib().cake_mixer_loop_rows(DT[a.dtype], _vec(x, "x", torch.float32),
+                                      _vec(x0, "x0", torch.float32, N * ld), ld,
+                                      _vec(step, "step", torch.float32, width), N, int(width), ap,
+                                      lda, _vec(y, "y", torch.float32, N * ld), _stream()),
+          "mixer_loop_rows")
+
+
+def gelu(x, out):
+    """out = erf GELU of x, f32 matrices with row strides."""
+    N, Fc = x.shape
+    xp, ldx = _mat(x, "x", torch.float32, N, Fc)
+    op, ldo = _mat(out, "out", torch.float32, N, Fc)
+    check(_lib().cake_mixer_gelu(xp, ldx, N, Fc, op, ldo, _stream()), "mixer_gelu")
+
+
+# ---------------------------------------------------------------------------
+# batch-1 decode projections (16-bit weights)
+# ---------------------------------------------------------------------------
+def layer_in(resid, norm_w, eps: float, offset: float, width: int, w, n_raw: int, out, act):
+    """One norm, every input projection: rows [0, n_raw) of w -> out f32, the rest ->
+    act = gelu(.) in w's dtype."""
+    N, K = w.shape
+    check(_lib().cake_mixer_in(DT[w.dtype], _vec(resid, "resid", torch.float32, K),
+                               _vec(norm_w, "norm_w", w.dtype, K), float(eps), float(offset),
+                               int(width), _vec(w, "w", w.dtype), K, N, int(n_raw),
+                               _vec(out, "out", torch.float32, n_raw),
+                               _vec(act, "act", w.dtype, N - n_raw), _stream()), "mixer_in")
+
+
+def layer_out(a, w, alpha: float, x, y):
+    """y = x + alpha W a (f32 x, y; y may be x)."""
+    N, K = w.shape
+    check(_lib().cake_mixer_out(DT[w.dtype], _vec(a, "a", w.dtype, K), _vec(w, "w", w.dtype), K, N,
+                                float(alpha), _vec(x, "x", torch.float32, N),
+                                _vec(y, "y", torch.float32, N), _stream()), "mixer_out")
+
+
+def loop_in(x, x0, step, w, width: int, y):
+    """y = W [x ; x0] + step (w [width, K >= 2 width], zero columns past 2 width)."""
+    N, K = w.shape
+    if N != width:
+        raise ValueError("loop_in: w needs one row per channel")
+    check(_lib().cake_mixer_loop(DT[w.dtype], _vec(x, "x", torch.float32, width),
+                                 _vec(x0, "x0", torch.float32, width),
+                                 _vec(step, "step", torch.float32, width),
+                                 _vec(w, "w", w.dtype), int(width), K,
+                                 _vec(y, "y", torch.float32, width), _stream()), "mixer_loop")
+
+
+# ---------------------------------------------------------------------------
+# attention
+# ---------------------------------------------------------------------------
+@dataclass(frozen=True)
+class AttnShape:
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    rot_pairs: int = 0
+
+    def __post_init__(self):
+        if self.heads % self.kv_heads or not 0 < self.dim <= MAX_HEAD or \
+                not 0 < self.vdim <= MAX_HEAD or 2 * self.rot_pairs > self.dim:
+            raise ValueError(f"unsupported attention shape {self}")
+
+    @property
+    def DP(self) -> int:
+        return pad_to(self.dim, 32)
+
+    @property
+    def DVP(self) -> int:
+        return pad_to(self.vdim, 16)
+
+    @property
+    def q_cols(self) -> int:
+        return self.heads * self.dim
+
+    @property
+    def qkv_cols(self) -> int:
+        return (self.heads + self.kv_heads) * self.dim + self.kv_heads * self.vdim
+
+    @property
+    def out_cols(self) -> int:
+        return self.heads * self.vdim
+
+    @property
+    def tiles(self) -> int:
+        """Workgroup columns of a decode launch: 16-row query tiles of every kv head."""
+        return self.kv_heads * (-(-(self.heads // self.kv_heads) // 16))
+
+    def part_floats(self, B: int, nsplit: int) -> int:
+        return B * self.tiles * nsplit * 16 * (self.DVP + 2)
+
+
+def _cache(sh: AttnShape, kc, vc, dtype):
+    """kc [slots, G, S, DP], vc [slots, G, DVP, S] -> (S, slots)."""
+    slots, G, S, DP = kc.shape
+    if (G, DP) != (sh.kv_heads, sh.DP) or tuple(vc.shape) != (slots, G, sh.DVP, S) or S % 64:
+        raise ValueError(f"cache shapes {tuple(kc.shape)} / {tuple(vc.shape)} do not fit {sh}")
+    for t in (kc, vc):
+        _vec(t, "cache", dtype)
+    return S, slots
+
+
+def _check_rows(rows: Rows, S: int, slots: int):
+    for _, n, p0, s in rows.host:
+        if not 0 <= s < slots or p0 < 0 or p0 + n > S:
+            raise ValueError(f"rows {p0}..{p0 + n} of slot {s} outside a {slots} x {S} cache")
+
+
+def attn_prep(sh: AttnShape, proj, rows: Rows, cs, qk_norm: bool, eps: float, qn, kc, vc):
+    """Rotate / normalise q (-> qn [N, H, DP]) and k, v (-> cache) of packed prompt rows."""
+    S, slots = _cache(sh, kc, vc, proj.dtype)
+    _check_rows(rows, S, slots)
+    pp, ldp = _mat(proj, "proj", proj.dtype, rows.N, sh.qkv_cols)
+    if sh.rot_pairs and (cs.shape[0] < S or cs.shape[1] != 2 * sh.rot_pairs):
+        raise ValueError("rotation table does not cover the cache")
+    check(_lib().cake_mixer_prep(DT[proj.dtype], pp, ldp, rows.N, sh.heads, sh.kv_heads, sh.dim,
+                                 sh.vdim, sh.DP, sh.DVP, S, sh.rot_pairs, int(qk_norm), float(eps),
+                                 _vec(cs, "cs", torch.float32), rows.pos.data_ptr(),
+                                 rows.slot.data_ptr(),
+                                 _vec(qn, "qn", proj.dtype, rows.N * sh.heads * sh.DP),
+                                 kc.data_ptr(), vc.data_ptr(), kc.stride(0), vc.stride(0),
+                                 _stream()), "mixer_prep")
+
+
+def attn_prompt(sh: AttnShape, qn, kc, vc, rows: Rows, gate, out, scale: float, sink: bool):
+    """Causal attention of packed rows over their sequences' caches; gate [N, H vdim] (pre
+    sigmoid) or None; out [N, >= H vdim]."""
+    S, slots = _cache(sh, kc, vc, qn.dtype)
+    _check_rows(rows, S, slots)
+    gp, ldg = (None, 0) if gate is None else _mat(gate, "gate", qn.dtype, rows.N, sh.out_cols)
+    op, ldo = _mat(out, "out", qn.dtype, rows.N, sh.out_cols)
+    check(_lib().cake_mixer_flash(DT[qn.dtype],
+                                  _vec(qn, "qn", qn.dtype, rows.N * sh.heads * sh.DP),
+                                  kc.data_ptr(), vc.data_ptr(), kc.stride(0), vc.stride(0),
+                                  _vec(rows.seq, "seq", torch.int32, 4 * rows.B), rows.B,
+                                  rows.max_len, gp, ldg, op, ldo, sh.heads, sh.kv_heads, sh.dim,
+                                  sh.vdim, sh.DP, sh.DVP, S, int(sink), float(scale), _stream()),
+          "mixer_flash")
+
+
+def attn_decode(sh: AttnShape, proj, pos, slot, cs, qk_norm: bool, sink: bool, gated: bool,
+                eps: float, scale: float, kc, vc, out, nsplit: int, part, ticket):
+    """One token per sequence: proj [B, q|k|v(|gate)] f32, pos / slot int32 [B] on the device
+    (the caller keeps pos < S); writes the new key / value and out [B, >= H vdim]."""
+    S, _ = _cache(sh, kc, vc, out.dtype)
+    B = proj.shape[0]
+    cols = sh.qkv_cols + (sh.out_cols if gated else 0)
+    pp, ldp = _mat(proj, "proj", torch.float32, B, cols)
+    op, ldo = _mat(out, "out", out.dtype, B, sh.out_cols)
+    if not 1 <= nsplit <= MAX_SPLIT:
+        raise ValueError(f"nsplit {nsplit} outside 1..{MAX_SPLIT}")
+    if sh.rot_pairs and (cs.shape[0] < S or cs.shape[1] != 2 * sh.rot_pairs):
+        raise ValueError("rotation table does not cover the cache")
+    check(_lib().cake_mixer_attn_decode(
+        DT[out.dtype], pp, ldp, B, _vec(pos, "pos", torch.int32, B),
+        _vec(slot, "slot", torch.int32, B), _vec(cs, "cs", torch.float32), sh.rot_pairs,
+        int(qk_norm), int(sink), int(gated), float(eps), float(scale), kc.data_ptr(),
+        vc.data_ptr(), kc.stride(0), vc.stride(0), op, ldo, sh.heads, sh.kv_heads, sh.dim,
+        sh.vdim, sh.DP, sh.DVP, S, int(nsplit),
+        _vec(part, "part", torch.float32, sh.part_floats(B, nsplit)),
+        _vec(ticket, "ticket", torch.int32, B * sh.tiles), _stream()), "mixer_attn_decode")
+
+
+# ---------------------------------------------------------------------------
+# gated delta rule
+# ---------------------------------------------------------------------------
+@dataclass(frozen=True)
+class DeltaShape:
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    taps: int
+
+    def __post_init__(self):
+        if self.heads % self.kv_heads or not 0 < self.dim <= MAX_HEAD or \
+                not 0 < self.vdim <= MAX_HEAD or self.taps < 1:
+            raise ValueError(f"unsupported delta-rule shape {self}")
+
+    @property
+    def EP(self) -> int:
+        return pad_to(self.vdim, 4)
+
+    @property
+    def channels(self) -> int:
+        return 2 * self.kv_heads * self.dim + self.heads * self.vdim
+
+    @property
+    def out_cols(self) -> int:
+        return self.heads * self.vdim
+
+
+def _delta_consts(sh: DeltaShape, conv, a_log, dt_bias, norm_w):
+    f = torch.float32
+    return (_vec(conv, "conv", f, sh.taps * sh.channels), _vec(a_log, "a_log", f, sh.heads),
+            _vec(dt_bias, "dt_bias", f, sh.heads), _vec(norm_w, "norm_w", f, sh.vdim))
+
+
+def _delta_state(sh: DeltaShape, state, ring):
+    if tuple(state.shape[1:]) != (sh.heads, sh.dim, sh.EP) or \
+            tuple(ring.shape[1:]) != (sh.taps, sh.channels) or state.shape[0] != ring.shape[0]:
+        raise ValueError(f"state shapes {tuple(state.shape)} / {tuple(ring.shape)} do not fit {sh}")
+    return (_vec(state, "state", torch.float32), _vec(ring, "ring", torch.float32),
+            state.stride(0), ring.stride(0))
+
+
+def delta_prompt(sh: DeltaShape, proj, ab, rows: Rows, eps: float, conv, a_log, dt_bias, norm_w,
+                 state, ring, out):
+    """Packed prompt rows: proj [N, q|k|v|gate], ab [N, a|b] f32 -> out [N, >= H vdim]; the
+    sequences' states advance."""
+    N, dev, f = rows.N, proj.device, torch.float32
+    _check_rows(rows, 1 << 30, state.shape[0])
+    pp, ldp = _mat(proj, "proj", proj.dtype, N, sh.channels + sh.out_cols)
+    abp, ldab = _mat(ab, "ab", f, N, 2 * sh.heads)
+    op, ldo = _mat(out, "out", proj.dtype, N, sh.out_cols)
+    G, H = sh.kv_heads, sh.heads
+    sizes = (N * G * sh.dim, N * G * sh.dim, N * H * sh.vdim, N * G, 2 * N * H, N * H * sh.vdim)
+    ws = torch.empty(sum(pad_to(s, 4) for s in sizes), device=dev, dtype=f)
+    ptrs, o = [], 0
+    for s in sizes:
+        ptrs.append(ws.data_ptr() + 4 * o)
+        o += pad_to(s, 4)
+    sp, rp, s_slot, r_slot = _delta_state(sh, state, ring)
+    check(_lib().cake_mixer_delta_prefill(
+        DT[proj.dtype], pp, ldp, abp, ldab, N, H, G, sh.dim, sh.vdim, sh.EP, sh.taps, float(eps),
+        *_delta_consts(sh, conv, a_log, dt_bias, norm_w), *ptrs, sp, rp, s_slot, r_slot,
+        rows.pos.data_ptr(), rows.slot.data_ptr(), rows.first.data_ptr(), rows.seq.data_ptr(),
+        rows.B, op, ldo, _stream()), "mixer_delta_prefill")
+
+
+def delta_decode(sh: DeltaShape, proj, ab, pos, slot, eps: float, conv, a_log, dt_bias, norm_w,
+                 state, ring, out):
+    """One token per sequence: proj [B, q|k|v|gate] f32, ab [B, a|b] f32."""
+    B, f = proj.shape[0], torch.float32
+    pp, ldp = _mat(proj, "proj", f, B, sh.channels + sh.out_cols)
+    abp, ldab = _mat(ab, "ab", f, B, 2 * sh.heads)
+    op, ldo = _mat(out, "out", out.dtype, B, sh.out_cols)
+    sp, rp, s_slot, r_slot = _delta_state(sh, state, ring)
+    check(_lib().cake_mixer_delta_decode(
+        DT[out.dtype], pp, ldp, abp, ldab, B, sh.heads, sh.kv_heads, sh.dim, sh.vdim, sh.EP,
+        sh.taps, float(eps), *_delta_consts(sh, conv, a_log, dt_bias, norm_w), sp, rp, s_slot,
+        r_slot, _vec(pos, "pos", torch.int32, B), _vec(slot, "slot", torch.int32, B), op, ldo,
+        _stream()), "mixer_delta_decode")
