@@ -130,15 +130,39 @@ def write_checkpoint(out_dir: str | Path, cfg: LlamaConfig, dtype: torch.dtype =
     return out
 
 
+def write_hybrid_checkpoint(out_dir: str | Path, config: dict, seed: int = 0) -> Path:
+    """A hybrid design (models/hybrid) with seeded random bf16 weights: config.json as given,
+    one model.safetensors, the synthetic tokenizer."""
+    from ..models.hybrid.config import from_config
+    from ..models.hybrid.weights import random_tensors, tensor_shapes
+    out = Path(out_dir)
+    out.mkdir(parents=True, exist_ok=True)
+    cfg = from_config(config)
+    (out / "config.json").write_text(json.dumps(config, indent=1))
+    if cfg.vocab_size < 256 + len(SPECIALS):
+        raise ValueError("the synthetic tokenizer needs a vocabulary of at least "
+                         f"{256 + len(SPECIALS)}")
+    write_tokenizer(out, cfg)
+    get = random_tensors(cfg, seed=seed)
+    save_file({n: get(n) for n in tensor_shapes(cfg)}, out / "model.safetensors",
+              {"format": "pt"})
+    return out
+
+
 def main(argv=None) -> int:
-    ap = argparse.ArgumentParser(description="write a random-init Llama-3 checkpoint")
+    ap = argparse.ArgumentParser(description="write a random-init checkpoint")
     ap.add_argument("--preset", default="tiny")
+    ap.add_argument("--config", default=None,
+                    help="config.json of a hybrid design (instead of a Llama preset)")
     ap.add_argument("--layers", type=int, default=None)
     ap.add_argument("--out", required=True)
     ap.add_argument("--dtype", default="bf16")
     ap.add_argument("--seed", type=int, default=0)
     ap.add_argument("--shard-mb", type=int, default=2048)
     a = ap.parse_args(argv)
+    if a.config:
+        print(write_hybrid_checkpoint(a.out, json.loads(Path(a.config).read_text()), a.seed))
+        return 0
     from ..models.llama3.factory import parse_dtype
     kw = {} if a.layers is None else {"num_hidden_layers": a.layers}
     cfg = tiny_config(**kw) if a.preset == "tiny" else preset(a.preset, **kw)
