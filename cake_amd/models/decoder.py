@@ -161,7 +161,7 @@ class DeviceDecoder:
         """The bucket graphs as the native decode loop's GraphSet (built once)."""
         gs = getattr(self, "_graph_set", None)
         if gs is None or gs.graphs[-1] is not self.graphs[max(self.graphs)]:
-            from ...ops import graph_loop as GL
+            from ..ops import graph_loop as GL
             caps = sorted(self.graphs)
             index = {c: i for i, c in enumerate(caps)}
             by_graph = {id(self.graphs[c]): index[c] for c in caps}

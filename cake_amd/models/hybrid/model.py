@@ -45,7 +45,7 @@ class DecodeState:
     xa: torch.Tensor       # residual rows: a looped pass is entered from one into the other
     xb: torch.Tensor
     proj: torch.Tensor     # [max n_raw] f32
-    act: torch.Tensor      # per layer run kind: [mixer output | feed-forward] storage dtype
+    act: torch.Tensor      # per layer: [mixer output | feed-forward], storage dtype
     part: torch.Tensor
     ticket: torch.Tensor
     pos: torch.Tensor
@@ -53,7 +53,7 @@ class DecodeState:
     tok: torch.Tensor
     hist: torch.Tensor
     hist_len: torch.Tensor
-    slot: torch.Tensor     # argmax key
+    slot: torch.Tensor     # token-selection key (argmax / draw)
     thr: torch.Tensor
     sel_ticket: torch.Tensor
     logits: torch.Tensor
@@ -77,7 +77,8 @@ class HybridModel:
         self.pool.length[GEN_SLOT] = 0
         self._rot: dict = {}
         self._none = torch.zeros(2, device=self.device)
-        self._bufs: DecodeState | None = None
+        self._bufs: DecodeState | None = None    # the captured decoder's
+        self._eager: DecodeState | None = None   # single-token steps of any sequence
         self._nsplit: int | None = None
         # decode attention's split partials and arrival tickets (zeroed once, re-armed by the
         # kernel); grown for the largest batch seen
@@ -238,16 +239,16 @@ class HybridModel:
         if len(seqs) == 1 and len(entries[0].tokens) == 1 and self.dtype != torch.float32 \
                 and observe is None:
             slot, pos, (tok,) = seqs[0]
-            b = self.decode_buffers()
+            if self._eager is None:  # not the captured decoder's: its step state lives on
+                self._eager = self._decode_buffers()
+            b = self._eager
             b.tok.fill_(tok)
             b.pos.fill_(pos)
             b.seq_slot.fill_(slot)
             self.decode_embed(b)
             with self.decode_eager(pos):
                 x = self.decode_layers(b, range(len(self.runs)))
-            out = self._logits(x.view(1, -1), [0] * len(entries[0].want))
-            b.seq_slot.fill_(GEN_SLOT)
-            return [out]
+            return [self._logits(x.view(1, -1), [0] * len(entries[0].want))]
         rows = M.Rows.pack(seqs, self.device)
         x = self._forward_rows(rows, observe)
         take = [h[0] + w for h, e in zip(rows.host, entries) for w in e.want]
@@ -280,18 +281,21 @@ class HybridModel:
 
     def decode_buffers(self) -> DecodeState:
         if self._bufs is None:
-            dev, f, i32 = self.device, torch.float32, torch.int32
-            z = partial(torch.zeros, device=dev)
-            part, ticket = self._split_ws(1)
-            self._bufs = DecodeState(
-                x0=z(self.Wp, dtype=f), xa=z(self.Wp, dtype=f), xb=z(self.Wp, dtype=f),
-                proj=z(max(w.n_raw for w in self.layers), dtype=f),
-                act=z((len(self.layers), max(w.out_cols for w in self.layers)), dtype=self.dtype),
-                part=part, ticket=ticket, pos=z(1, dtype=i32), seq_slot=z(1, dtype=i32),
-                tok=z(1, dtype=i32), hist=z(self.max_seq, dtype=i32), hist_len=z(1, dtype=i32),
-                slot=z(1, dtype=torch.int64), thr=z(1, dtype=i32), sel_ticket=z(1, dtype=i32),
-                logits=z(self.cfg.vocab_size, dtype=f))
+            self._bufs = self._decode_buffers()
         return self._bufs
+
+    def _decode_buffers(self) -> DecodeState:
+        f, i32 = torch.float32, torch.int32
+        z = partial(torch.zeros, device=self.device)
+        part, ticket = self._split_ws(1)
+        return DecodeState(
+            x0=z(self.Wp, dtype=f), xa=z(self.Wp, dtype=f), xb=z(self.Wp, dtype=f),
+            proj=z(max(w.n_raw for w in self.layers), dtype=f),
+            act=z((len(self.layers), max(w.out_cols for w in self.layers)), dtype=self.dtype),
+            part=part, ticket=ticket, pos=z(1, dtype=i32), seq_slot=z(1, dtype=i32),
+            tok=z(1, dtype=i32), hist=z(self.max_seq, dtype=i32), hist_len=z(1, dtype=i32),
+            slot=z(1, dtype=torch.int64), thr=z(1, dtype=i32), sel_ticket=z(1, dtype=i32),
+            logits=z(self.cfg.vocab_size, dtype=f))
 
     def decode_state(self, b: DecodeState) -> list[torch.Tensor]:
         return [b.tok, b.pos, b.hist_len, b.x0, *self.pool.recurrent(GEN_SLOT)]
@@ -368,4 +372,3 @@ class HybridModel:
     def prefill_logits(self, prompt: list[int], out: torch.Tensor) -> None:
         self.reset()
         out.copy_(self.forward(prompt, 0))
-        self.decode_buffers().seq_slot.fill_(GEN_SLOT)
