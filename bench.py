@@ -101,7 +101,25 @@ def _args(argv=None):
                          "torchrun roles); python = the torch-hosted decoders (test oracles)")
     ap.add_argument("--launch-timeout", type=float, default=1800.0,
                     help="self-launch (N>1 without torchrun): kill the ranks after this many s")
+    ap.add_argument("--design", default=None, choices=["fonapel"],
+                    help="instead of the headline: prefill and decode throughput of a hybrid "
+                         "design beside Llama layers of equal size, one JSON line per size")
+    ap.add_argument("--design-sizes", default="w2048,w4096,w8192")
+    ap.add_argument("--design-models", default="hybrid,llama",
+                    help="which of the two to run (profiling)")
     return ap.parse_args(argv)
+
+
+def bench_design(a) -> None:
+    """--design: models/hybrid/bench.py at each size."""
+    from cake_amd.models.hybrid.bench import measure
+    from cake_amd.models.llama3.factory import parse_dtype
+    torch.cuda.set_device(0)
+    for size in a.design_sizes.split(","):
+        r = measure(size, parse_dtype(a.dtype), which=tuple(a.design_models.split(",")))
+        print(json.dumps({"metric": "design_throughput", "design": a.design, "size": size,
+                          "data": "synthetic (random-init weights, synthetic prompt ids)", **r}),
+              flush=True)
 
 
 def _emit(a, value, ms, p50, p99, n, extra):
@@ -443,6 +461,9 @@ def self_launch(a, argv) -> int:
 def main(argv=None) -> int:
     argv = list(sys.argv[1:] if argv is None else argv)
     a = _args(argv)
+    if a.design:
+        bench_design(a)
+        return 0
     world = int(os.environ.get("WORLD_SIZE", "1"))
     if a.gpus > 1 and "WORLD_SIZE" not in os.environ:
         return self_launch(a, argv)

@@ -1,0 +1,120 @@
+"""Throughput of a hybrid design beside Llama layers of equal size (bench.py --design).
+
+Sizes follow the layers of real models.  Per size the hybrid model has six layers (attention
+and delta, a looped section of three run twice: nine layer runs, all mechanisms) and the
+Llama model nine layers of the same width, heads and head size; the feed-forward widths make
+an attention layer of one as many parameters as a layer of the other.  Random-init weights.
+"""
+from __future__ import annotations
+
+import gc
+import time
+
+import torch
+
+from .config import AttentionMixer, DeltaMixer, DenseMlp, HybridConfig, Layer, Loop, Rotary
+
+SIZES = {  # width, heads, kv heads, Llama feed-forward, vocabulary
+    "w2048": (2048, 16, 4, 8192, 32000),
+    "w4096": (4096, 32, 8, 14336, 32000),
+    "w8192": (8192, 64, 8, 28672, 32000),
+}
+DIM = 128
+
+
+def hybrid_config(size: str) -> HybridConfig:
+    W, H, G, ff, V = SIZES[size]
+    attn = AttentionMixer(H, G, DIM, DIM, scale=DIM ** -0.5, rot=Rotary(64, 5e5))
+    delta = DeltaMixer(H, H // 2, DIM, DIM, taps=4)
+    # llama: 2 W^2 + 2 W G d + 3 W ff; here one W^2 more (the gate) and two of three ff matrices
+    mlp = DenseMlp((3 * ff - H * DIM) // 2)
+    return HybridConfig("fonapel", V, W, [Layer(m, mlp) for m in
+                                          (attn, delta, attn, attn, delta, attn)], eps=1e-5,
+                        residual_mult=0.5, loop=Loop(1, 4, 2))
+
+
+def llama_config(size: str):
+    from ..llama3.config import LlamaConfig
+    W, H, G, ff, V = SIZES[size]
+    return LlamaConfig(hidden_size=W, intermediate_size=ff, vocab_size=V, num_hidden_layers=9,
+                       num_attention_heads=H, num_key_value_heads=G, rope_theta=5e5)
+
+
+def _params(cfg) -> int:
+    if isinstance(cfg, HybridConfig):
+        from .weights import tensor_shapes
+        return sum(torch.Size(s).numel() for s in tensor_shapes(cfg).values())
+    return cfg.num_hidden_layers * cfg.layer_bytes(1) + 2 * cfg.vocab_size * cfg.hidden_size
+
+
+def _step_weights(cfg: HybridConfig) -> int:
+    """Weight elements one decoded token reads (a looped layer once per pass)."""
+    from .weights import tensor_shapes
+    by_layer, rest = {}, 0
+    for n, s in tensor_shapes(cfg).items():
+        k = torch.Size(s).numel()
+        if n.startswith("l") and n[1].isdigit():
+            i = int(n[1:n.index(".")])
+            by_layer[i] = by_layer.get(i, 0) + k
+        elif n == "loop.in":
+            rest += k * cfg.loop.times
+        elif n == "head":
+            rest += k
+    return rest + sum(by_layer[r.layer] for r in cfg.runs())
+
+
+def _measure(model, prompt_len: int, decode_at: int, steps: int, reps: int) -> dict:
+    from ..decoder import DeviceDecoder
+    from ..llama3.decode_loop import run_decode
+    g = torch.Generator().manual_seed(7)
+    ids = torch.randint(0, model.cfg.vocab_size, (max(prompt_len, decode_at),), generator=g).tolist()
+    buf = torch.empty(model.cfg.vocab_size, device="cuda", dtype=torch.float32)
+    model.prefill_logits(ids[:prompt_len], buf)
+    torch.cuda.synchronize()
+    times = []
+    for _ in range(reps):
+        t0 = time.perf_counter()
+        model.prefill_logits(ids[:prompt_len], buf)
+        torch.cuda.synchronize()
+        times.append(time.perf_counter() - t0)
+    pre = sorted(times)[len(times) // 2]
+    out = {"prefill_tokens_per_sec": round(prompt_len / pre, 1), "prefill_ms": round(pre * 1e3, 3)}
+    dec = DeviceDecoder(model, repeat_penalty=1.0)
+    for at in (32, decode_at):
+        dec.start(ids[:at])
+        dec.capture()
+        run_decode(dec, 8)
+        st = run_decode(dec, steps)
+        torch.cuda.synchronize()
+        out[f"decode_tokens_per_sec_at_{at}"] = round(len(st.tokens) / st.wall_s, 1)
+        out[f"decode_us_at_{at}"] = round(st.percentile(50) * 1e3, 1)
+    return out
+
+
+def measure(size: str, dtype=torch.bfloat16, prompt_len: int = 2048, decode_at: int = 2048,
+            steps: int = 64, reps: int = 5, which=("hybrid", "llama")) -> dict:
+    from ..llama3.factory import random_model
+    from .model import HybridModel
+    from .weights import random_tensors
+    max_seq = max(prompt_len, decode_at) + steps + 64
+    hc, lc = hybrid_config(size), llama_config(size)
+    out: dict = {"prompt_len": prompt_len, "dtype": str(dtype).split(".")[-1]}
+    for name in which:
+        if name == "hybrid":
+            m = HybridModel.build(hc, random_tensors(hc, "cuda", dtype), "cuda", dtype, max_seq)
+            n = _step_weights(hc)
+        else:
+            m = random_model(lc, "cuda", dtype, max_seq=max_seq)
+            n = _params(lc) - lc.vocab_size * lc.hidden_size
+        r = _measure(m, prompt_len, decode_at, steps, reps)
+        r["layer_runs"] = m.num_decode_layers
+        r["step_weight_gb"] = round(n * 2 / 1e9, 3)
+        r["decode_tb_per_s_at_32"] = round(n * 2 / r["decode_us_at_32"] / 1e6, 3)
+        out[name] = r
+        del m
+        gc.collect()
+        torch.cuda.empty_cache()
+    if len(which) == 2:
+        out["ratio"] = {k: round(out["hybrid"][k] / out["llama"][k], 3)
+                        for k in out["hybrid"] if k.endswith("per_sec") or "per_sec_at" in k}
+    return out
