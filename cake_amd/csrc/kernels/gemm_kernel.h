@@ -25,9 +25,21 @@ enum GemmEpi : int {
 };
 
 // the activation of kEpiSilu (runtime-uniform: one kernel instance for all three)
+// erf by Abramowitz & Stegun, formula 7.1.26 (|error| <= 1.5e-7): one exponential, one
+// reciprocal and a polynomial, no branch — the epilogue evaluates it once per output, where
+// erff's branches stood out (the result is rounded to 16 bits)
+__device__ __forceinline__ float erf_as(float x) {
+  const float ax = fabsf(x), t = __builtin_amdgcn_rcpf(fmaf(0.3275911f, ax, 1.f));
+  float p = fmaf(1.061405429f, t, -1.453152027f);
+  p = fmaf(p, t, 1.421413741f);
+  p = fmaf(p, t, -0.284496736f);
+  p = fmaf(p, t, 0.254829592f);
+  return copysignf(fmaf(-p * t, __expf(-ax * ax), 1.f), x);
+}
+
 __device__ __forceinline__ float gemm_act(int act, float x) {
   if (act == 1) return x * __frcp_rn(1.f + __expf(-1.702f * x));  // quick_gelu
-  if (act == 2) return 0.5f * x * (1.f + erff(x * 0.70710678118654752f));  // GELU (erf)
+  if (act == 2) return 0.5f * x * (1.f + erf_as(x * 0.70710678118654752f));  // GELU (erf)
   return silu(x);
 }
 

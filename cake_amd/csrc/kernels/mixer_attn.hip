@@ -39,7 +39,7 @@ struct PrepArgs {
 
 // LPH lanes per (row, head), four consecutive dims each
 template <int DT>
-__global__ __launch_bounds__(256) void mixer_prep_qk_kernel(PrepArgs a, int lph) {
+__global__ __launch_bounds__(256) void mixer_prep_qk_kernel(PrepArgs a, int lph, int vec) {
   using E = typename St<DT>::E;
   const int per = 256 / lph;  // (row, head) items per workgroup
   const int item = blockIdx.x * per + threadIdx.x / lph;
@@ -51,8 +51,14 @@ __global__ __launch_bounds__(256) void mixer_prep_qk_kernel(PrepArgs a, int lph)
   const int pos = a.row_pos[n];
   const E* src = reinterpret_cast<const E*>(a.proj) + (long long)n * a.ldp + (long long)hh * a.dim;
   float x[4];
+  if (DT != kF32 && vec) {  // rows and heads on 8-byte boundaries, dim % 4 == 0
+    const uint2 w = d0 < a.dim ? *reinterpret_cast<const uint2*>(src + d0) : make_uint2(0u, 0u);
+    x[0] = St<DT>::ld((uint16_t)(w.x & 0xffffu)); x[1] = St<DT>::ld((uint16_t)(w.x >> 16));
+    x[2] = St<DT>::ld((uint16_t)(w.y & 0xffffu)); x[3] = St<DT>::ld((uint16_t)(w.y >> 16));
+  } else {
 #pragma unroll
-  for (int e = 0; e < 4; ++e) x[e] = d0 + e < a.dim ? St<DT>::ld(src[d0 + e]) : 0.f;
+    for (int e = 0; e < 4; ++e) x[e] = d0 + e < a.dim ? St<DT>::ld(src[d0 + e]) : 0.f;
+  }
 #pragma unroll
   for (int p = 0; p < 2; ++p) {
     const int i = 2 * l + p;
@@ -427,11 +433,17 @@ __global__ __launch_bounds__(64 * kDecWaves) void mixer_attn_decode_kernel(MixDe
   };
   int k0 = kbeg + 32 * wave;
   if (kPrefetch && k0 < klim) { load_k(k0); load_vs(k0); }
+  // this thread's first two gate values, first needed at the very end
+  const float* gate = pj + (long long)(a.H + a.G) * a.dim + (long long)a.G * a.vdim +
+                      (long long)(hk * R + r0) * a.vdim;
+  float gpre[2] = {0.f, 0.f};
+  if (a.gated)
+#pragma unroll
+    for (int i = 0; i < 2; ++i)
+      if (tid + 64 * kDecWaves * i < nr * a.vdim) gpre[i] = gate[tid + 64 * kDecWaves * i];
 
-  for (int i = tid; i < 16 * (CLS + EPC); i += 64 * kDecWaves) qs[i] = E(0);
-  if (owner)
-    for (int i = tid; i < CLS; i += 64 * kDecWaves) { kcur[i] = E(0); vcur[i] = E(0); }
-  __syncthreads();
+  // rows past nr and value columns past vdim stay unwritten: they only reach accumulator
+  // columns / rows that no output reads
   for (int r = wave; r < nr + (owner ? 1 : 0); r += kDecWaves) {
     const bool isk = r == nr;
     const float* src = isk ? pj + (long long)(a.H + hk) * a.dim
@@ -441,7 +453,7 @@ __global__ __launch_bounds__(64 * kDecWaves) void mixer_attn_decode_kernel(MixDe
     E* dst = isk ? kcur : qs + r * (CLS + EPC);
 #pragma unroll
     for (int e = 0; e < 4; ++e)
-      if (4 * lane + e < a.dim) dst[4 * lane + e] = St<DT>::st(x[e]);
+      if (4 * lane + e < DP) dst[4 * lane + e] = St<DT>::st(x[e]);  // zeros past dim
   }
   if (owner) {
     const float* vsrc = pj + (long long)(a.H + a.G) * a.dim + (long long)hk * a.vdim;
@@ -537,13 +549,12 @@ __global__ __launch_bounds__(64 * kDecWaves) void mixer_attn_decode_kernel(MixDe
   const int ngt = gridDim.x;
   const long long pstride = 16ll * (DVP + 2);
   float* part = a.part + ((long long)b * ngt + gt) * a.nsplit * pstride;
-  auto finish = [&](int r, int d, float num, float den) {
+  E* out = reinterpret_cast<E*>(a.out) + (long long)b * a.ldo + (long long)(hk * R + r0) * a.vdim;
+  auto finish = [&](int i, float num, float den) {  // i = r vdim + d: heads are contiguous
     float y = num / den;
-    const int hh = hk * R + r0 + r;
     if (a.gated)
-      y *= sigmoid32(pj[(long long)(a.H + a.G) * a.dim + (long long)a.G * a.vdim +
-                        (long long)hh * a.vdim + d]);
-    reinterpret_cast<E*>(a.out)[(long long)b * a.ldo + (long long)hh * a.vdim + d] = St<DT>::st(y);
+      y *= sigmoid32(i < 64 * kDecWaves ? gpre[0] : i < 128 * kDecWaves ? gpre[1] : gate[i]);
+    out[i] = St<DT>::st(y);
   };
   for (int i = tid; i < nr * a.vdim; i += 64 * kDecWaves) {
     const int r = i / a.vdim, d = i - r * a.vdim;
@@ -559,7 +570,7 @@ __global__ __launch_bounds__(64 * kDecWaves) void mixer_attn_decode_kernel(MixDe
       den = fmaf(f, red_l[w][r], den);
     }
     if (nact == 1) {
-      finish(r, d, num, den);
+      finish(i, num, den);
     } else {
       float* pr = part + sp * pstride + (long long)r * (DVP + 2);
       // agent-scope stores: the merging workgroup may run on another XCD
@@ -571,34 +582,57 @@ __global__ __launch_bounds__(64 * kDecWaves) void mixer_attn_decode_kernel(MixDe
     }
   }
   if (nact == 1) return;
-  // the last split to arrive merges all of them
-  __threadfence();
+  // the last split to arrive merges all of them: every wave's partials are out before the
+  // workgroup's arrival counts, and both sides use agent-scope accesses
+  asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
   __syncthreads();
   if (tid == 0) {
     unsigned int* tk = a.ticket + (long long)b * ngt + gt;
     const unsigned int old =
-        __hip_atomic_fetch_add(tk, 1u, __ATOMIC_ACQ_REL, __HIP_MEMORY_SCOPE_AGENT);
+        __hip_atomic_fetch_add(tk, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
     s_last = old == (unsigned int)(nact - 1);
     if (s_last) __hip_atomic_store(tk, 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
   }
   __syncthreads();
   if (!s_last) return;
-  __threadfence();
+  float* wm = &red_o[0][0][0];      // [nact][16] max -> weight; the wave partials are spent
+  float* wl = wm + 16 * 64;         // [nact][16] sums
+  float* wd = &red_m[0][0];         // [16] denominators
+  static_assert(sizeof(red_o) >= 2 * 16 * 64 * sizeof(float), "merge scratch");
+  for (int i = tid; i < nr * nact; i += 64 * kDecWaves) {
+    const int s = i / nr, r = i - s * nr;
+    const float* pr = part + s * pstride + (long long)r * (DVP + 2);
+    wm[s * 16 + r] = __hip_atomic_load(pr, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    wl[s * 16 + r] = __hip_atomic_load(pr + 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+  }
+  __syncthreads();
+  if (tid < nr) {
+    float M = a.sink ? 0.f : -INFINITY;
+    for (int s = 0; s < nact; ++s) M = fmaxf(M, wm[s * 16 + tid]);
+    float den = a.sink ? __builtin_amdgcn_exp2f(-M) : 0.f;
+    for (int s = 0; s < nact; ++s) {
+      const float f = __builtin_amdgcn_exp2f(wm[s * 16 + tid] - M);
+      den = fmaf(f, wl[s * 16 + tid], den);
+      wm[s * 16 + tid] = f;
+    }
+    wd[tid] = den;
+  }
+  __syncthreads();
   for (int i = tid; i < nr * a.vdim; i += 64 * kDecWaves) {
     const int r = i / a.vdim, d = i - r * a.vdim;
-    const float* pr = part + (long long)r * (DVP + 2);
-    float M = a.sink ? 0.f : -INFINITY;
-    for (int s = 0; s < nact; ++s)
-      M = fmaxf(M, __hip_atomic_load(pr + s * pstride, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT));
-    float num = 0.f, den = a.sink ? __builtin_amdgcn_exp2f(-M) : 0.f;
-    for (int s = 0; s < nact; ++s) {
-      const float* ps = pr + s * pstride;
-      const float f = __builtin_amdgcn_exp2f(
-          __hip_atomic_load(ps, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) - M);
-      num = fmaf(f, __hip_atomic_load(ps + 2 + d, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT), num);
-      den = fmaf(f, __hip_atomic_load(ps + 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT), den);
+    const float* pr = part + (long long)r * (DVP + 2) + 2 + d;
+    float num = 0.f;
+    for (int s0 = 0; s0 < nact; s0 += 8) {  // eight partials in flight
+      float v[8];
+#pragma unroll
+      for (int j = 0; j < 8; ++j)
+        v[j] = __hip_atomic_load(pr + min(s0 + j, nact - 1) * pstride, __ATOMIC_RELAXED,
+                                 __HIP_MEMORY_SCOPE_AGENT);
+#pragma unroll
+      for (int j = 0; j < 8; ++j)
+        if (s0 + j < nact) num = fmaf(wm[(s0 + j) * 16 + r], v[j], num);
     }
-    finish(r, d, num, den);
+    finish(i, num, wd[r]);
   }
 }
 
@@ -623,10 +657,11 @@ CAKE_API int cake_mixer_prep(int dt, const void* proj, long long ldp, int N, int
              row_pos, row_slot, qn, kc, vc, k_slot, v_slot};
   int lph = 8;
   while (4 * lph < DP) lph <<= 1;  // <= 64
+  const int vec = dim % 4 == 0 && ldp % 4 == 0 && ((uintptr_t)proj % 8) == 0;
   const long long items = (long long)N * (H + G);
   const dim3 g1((unsigned)((items + 256 / lph - 1) / (256 / lph)));
   const dim3 g2((N + 63) / 64, (G * ((vdim + 7) / 8) + 3) / 4);
-  CAKE_MIX_DT(dt, hipLaunchKernelGGL((mixer_prep_qk_kernel<DT>), g1, dim3(256), 0, st, a, lph);
+  CAKE_MIX_DT(dt, hipLaunchKernelGGL((mixer_prep_qk_kernel<DT>), g1, dim3(256), 0, st, a, lph, vec);
               hipLaunchKernelGGL((mixer_prep_v_kernel<DT>), g2, dim3(256), 0, st, a));
   return (int)hipGetLastError();
 }

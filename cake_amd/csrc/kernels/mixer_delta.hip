@@ -9,11 +9,19 @@
 // the same step still reads).  A sequence at position 0 starts from zeros whatever its slot
 // held before.
 //
-//   * mixer_delta_prep (prompt rows): convolution, SiLU, unit norms, q.k, step size, decay.
-//   * mixer_delta_scan: the recurrence of one sequence.  The columns of S are independent
-//     given k, q, the decay and the step size, so a workgroup takes 16 columns of one head:
-//     16 lanes hold one column in registers, dot products are in-row DPP sums, and the
-//     read-out uses o = decay (S^T q) + (q.k) u, so both dots run side by side ahead of u.
+// Prompt rows run in chunks of 16 tokens.  Inside a chunk (decay products G_ij over tokens
+// j+1..i, g_i from the chunk's start), with the chunk's entry state S0:
+//     (I + A) U = R,  A_ij = beta_i G_ij (k_i.k_j) for j < i,  R_i = beta_i (v_i - g_i S0^T k_i)
+//     o_i = g_i S0^T q_i + sum_{j <= i} G_ij (q_i.k_j) u_j
+//     S   = g_15 S0 + sum_j G_15,j k_j u_j^T
+// so everything is 16-row f32 matrix products (v_mfma_f32_16x16x4_f32) except the small
+// triangular inverse, which does not depend on the state.
+//
+//   * mixer_delta_prep: convolution, SiLU and unit norms of a chunk's rows.
+//   * mixer_delta_chunk: per chunk and head T = (I + A)^-1, P_ij = G_ij (q_i.k_j), g, beta.
+//   * mixer_delta_scan: walks the chunks of one sequence.  A workgroup takes 16 columns of one
+//     head's S; its four waves hold a quarter of the rows each, as accumulators that are the
+//     next chunk's B operands; the partial S0^T k, S0^T q meet in LDS once per chunk.
 //   * mixer_delta_out: gated norm of the read-outs.
 //   * mixer_delta_decode: all of it for one token per sequence in one launch.
 #include "mixer_common.h"
@@ -31,11 +39,12 @@ struct DeltaArgs {
   const float* a_log;     // [H] f32
   const float* dt_bias;   // [H] f32
   const float* norm_w;    // [vdim] f32
-  float* qn;              // [N][G][dim]
-  float* kn;              // [N][G][dim]
+  int DR;                 // dim padded to 64
+  float* qn;              // [N][G][DR], zeros past dim
+  float* kn;              // [N][G][DR]
   float* vv;              // [N][H][vdim]
-  float* qk;              // [N][G]
-  float* bd;              // [N][H][2] (decay, beta)
+  float* tp;              // [NC][H][2][16][16]: T, P
+  float* gm;              // [NC][H][16][4]: g_i, beta_i, G_15,i, g_15
   float* o;               // [N][H][vdim]
   float* state;
   float* ring;
@@ -44,6 +53,9 @@ struct DeltaArgs {
   const int* row_slot;    // [N]
   const int* row_seq0;    // [N] packed row of the sequence's first token in this step
   const SeqRow* seq;      // [B]
+  const int2* chunk;      // [NC]: packed row of the first token, tokens
+  const int* chunk0;      // [B]: first chunk of the sequence
+  int NC;
   void* out;              // [N][ldo]
   long long ldo;
 };
@@ -52,178 +64,275 @@ __device__ __forceinline__ int delta_channels(const DeltaArgs& a) {
   return 2 * a.G * a.dim + a.H * a.vdim;
 }
 
-// convolution + SiLU of channel c at packed row n (prompt rows)
+// the raw projection of channel c, `back` tokens before packed row n at position pos
 template <int DT>
-__device__ __forceinline__ float conv_row(const DeltaArgs& a, int n, int pos, int first, int c,
-                                          const float* ring, int C) {
+__device__ __forceinline__ float conv_tap(const DeltaArgs& a, int n, int pos, int first, int back,
+                                          int c, const float* ring, int C) {
+  if (pos < back) return 0.f;
+  if (n - back >= first)
+    return St<DT>::ld(reinterpret_cast<const typename St<DT>::E*>(a.proj)[(long long)(n - back) *
+                                                                             a.ldp + c]);
+  return ring[(long long)((pos - back) % a.taps) * C + c];
+}
+
+constexpr int kChunk = 16;
+constexpr int kWin = 8;  // taps a lane keeps in registers
+
+// A wave per (chunk, unit): units [0, 2G) the q and k heads, [2G, 2G + H) the value heads;
+// CPL consecutive channels per lane, the last kWin inputs of each in registers.
+template <int DT, int CPL>
+__global__ __launch_bounds__(256) void mixer_delta_prep_kernel(DeltaArgs a, int vec) {
   using E = typename St<DT>::E;
-  const E* x = reinterpret_cast<const E*>(a.proj) + c;
-  float y = 0.f;
-  for (int j = 0; j < a.taps; ++j) {  // j tokens back
-    const int p = pos - j;
-    if (p < 0) break;
-    const int src = n - j;
-    const float v = src >= first ? St<DT>::ld(x[(long long)src * a.ldp])
-                                 : ring[(long long)(p % a.taps) * C + c];
-    y = fmaf(a.conv[(long long)(a.taps - 1 - j) * C + c], v, y);
-  }
-  return silu32(y);
-}
-
-// a wave per (row, unit): units [0, G) = the q and k of one head, [G, G + H) = one value head
-template <int DT>
-__global__ __launch_bounds__(256) void mixer_delta_prep_kernel(DeltaArgs a) {
   const int lane = threadIdx.x & 63;
-  const int units = a.G + a.H;
+  const int units = 2 * a.G + a.H;
   const long long item = (long long)blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (item >= (long long)a.N * units) return;
-  const int n = (int)(item / units), u = (int)(item - (long long)n * units);
+  if (item >= (long long)a.NC * units) return;
+  const int ch = (int)(item / units), u = (int)(item - (long long)ch * units);
   const int C = delta_channels(a);
-  const int pos = a.row_pos[n], first = a.row_seq0[n];
-  const float* ring = a.ring + a.row_slot[n] * a.r_slot;
-  if (u < a.G) {
-    float q[4], k[4];
-    float sq = 0.f, sk = 0.f, qk = 0.f;
+  const int n0 = a.chunk[ch].x, cnt = a.chunk[ch].y;
+  const int pos0 = a.row_pos[n0], first = a.row_seq0[n0];
+  const float* ring = a.ring + a.row_slot[n0] * a.r_slot;
+  const bool isv = u >= 2 * a.G;
+  const int size = isv ? a.vdim : a.dim;
+  const int cb = isv ? 2 * a.G * a.dim + (u - 2 * a.G) * a.vdim : u * a.dim;
+  const int c0 = CPL * lane;
+  float* out = isv ? a.vv + (u - 2 * a.G) * a.vdim
+                   : (u < a.G ? a.qn + u * a.DR : a.kn + (u - a.G) * a.DR);
+  const long long ostride = isv ? (long long)a.H * a.vdim : (long long)a.G * a.DR;
+  const int osize = isv ? a.vdim : a.DR;
+  const float qs = u < a.G ? 1.f / sqrtf((float)a.dim) : 1.f;
+
+  float w[kWin][CPL], win[kWin][CPL];
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int d = lane + 64 * i;
-      q[i] = k[i] = 0.f;
-      if (d < a.dim) {
-        q[i] = conv_row<DT>(a, n, pos, first, u * a.dim + d, ring, C);
-        k[i] = conv_row<DT>(a, n, pos, first, (a.G + u) * a.dim + d, ring, C);
+  for (int j = 0; j < kWin; ++j)
+#pragma unroll
+    for (int e = 0; e < CPL; ++e) {
+      const bool ok = j < a.taps && c0 + e < size;
+      w[j][e] = ok ? a.conv[(long long)(a.taps - 1 - j) * C + cb + c0 + e] : 0.f;
+      // input j tokens before row 0 lives at index (0 - j) & 7
+      win[(kWin - j) & (kWin - 1)][e] =
+          ok && j > 0 ? conv_tap<DT>(a, n0, pos0, first, j, cb + c0 + e, ring, C) : 0.f;
+    }
+  const E* src = reinterpret_cast<const E*>(a.proj) + (long long)n0 * a.ldp + cb + c0;
+#pragma unroll
+  for (int t = 0; t < kChunk; ++t) {
+    if (t < cnt) {  // wave-uniform
+      float x[CPL];
+      if constexpr (CPL == 2 && DT != kF32) {
+        if (vec && c0 + 1 < size) {
+          const uint32_t p = *reinterpret_cast<const uint32_t*>(src + (long long)t * a.ldp);
+          x[0] = St<DT>::ld((uint16_t)(p & 0xffffu));
+          x[1] = St<DT>::ld((uint16_t)(p >> 16));
+        } else {
+#pragma unroll
+          for (int e = 0; e < CPL; ++e)
+            x[e] = c0 + e < size ? St<DT>::ld(src[(long long)t * a.ldp + e]) : 0.f;
+        }
+      } else {
+#pragma unroll
+        for (int e = 0; e < CPL; ++e)
+          x[e] = c0 + e < size ? St<DT>::ld(src[(long long)t * a.ldp + e]) : 0.f;
       }
-      sq += q[i] * q[i];
-      sk += k[i] * k[i];
-    }
-    const float rq = 1.f / sqrtf(wave_sum(sq) + 1e-6f) / sqrtf((float)a.dim);
-    const float rk = 1.f / sqrtf(wave_sum(sk) + 1e-6f);
-    float* qo = a.qn + ((long long)n * a.G + u) * a.dim;
-    float* ko = a.kn + ((long long)n * a.G + u) * a.dim;
+      float y[CPL], ss = 0.f;
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int d = lane + 64 * i;
-      q[i] *= rq;
-      k[i] *= rk;
-      qk += q[i] * k[i];
-      if (d < a.dim) { qo[d] = q[i]; ko[d] = k[i]; }
-    }
-    qk = wave_sum(qk);
-    if (lane == 0) a.qk[(long long)n * a.G + u] = qk;
-  } else {
-    const int h = u - a.G;
-    for (int d = lane; d < a.vdim; d += 64)
-      a.vv[((long long)n * a.H + h) * a.vdim + d] =
-          conv_row<DT>(a, n, pos, first, 2 * a.G * a.dim + h * a.vdim + d, ring, C);
-    if (lane == 0) {
-      const float* ab = a.ab + (long long)n * a.ldab;
-      float* bd = a.bd + ((long long)n * a.H + h) * 2;
-      bd[0] = expf(-expf(a.a_log[h]) * softplus32(ab[h] + a.dt_bias[h]));
-      bd[1] = sigmoid32(ab[a.H + h]);
+      for (int e = 0; e < CPL; ++e) {
+        win[t & (kWin - 1)][e] = x[e];
+        y[e] = 0.f;
+#pragma unroll
+        for (int j = 0; j < kWin; ++j) y[e] = fmaf(w[j][e], win[(t - j) & (kWin - 1)][e], y[e]);
+        if (a.taps > kWin)  // longer convolutions: the older inputs from memory
+          for (int j = kWin; j < a.taps; ++j)
+            if (c0 + e < size)
+              y[e] = fmaf(a.conv[(long long)(a.taps - 1 - j) * C + cb + c0 + e],
+                          conv_tap<DT>(a, n0 + t, pos0 + t, first, j, cb + c0 + e, ring, C), y[e]);
+        y[e] = silu32(y[e]);
+        ss += y[e] * y[e];
+      }
+      const float r = isv ? 1.f : qs / sqrtf(wave_sum(ss) + 1e-6f);
+      float* o = out + (long long)(n0 + t) * ostride + c0;
+      if constexpr (CPL == 2) {
+        if (c0 + 1 < osize && (osize & 1) == 0) {
+          *reinterpret_cast<float2*>(o) = make_float2(y[0] * r, y[1] * r);
+          continue;
+        }
+      }
+#pragma unroll
+      for (int e = 0; e < CPL; ++e)
+        if (c0 + e < osize) o[e] = y[e] * r;
     }
   }
 }
 
-constexpr int kScanTok = 16;  // tokens staged per round
+// grid (NC, G), 256 threads: the state-independent matrices of every head of a group
+__global__ __launch_bounds__(256) void mixer_delta_chunk_kernel(DeltaArgs a) {
+  __shared__ float kk[16][17], qk[16][17], am[16][16][17];
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, l15 = lane & 15, g = lane >> 4;
+  const int ch = blockIdx.x, gh = blockIdx.y;
+  const int n0 = a.chunk[ch].x, cnt = a.chunk[ch].y;
+  if (wave < 2) {  // k.k and q.k: rows past the chunk's end repeat the last, masked below
+    const int row = n0 + min(l15, cnt - 1);
+    const float* kp = a.kn + ((long long)row * a.G + gh) * a.DR + 4 * g;
+    const float* xp = (wave == 0 ? a.kn : a.qn) + ((long long)row * a.G + gh) * a.DR + 4 * g;
+    cf32x4 acc{0.f, 0.f, 0.f, 0.f};
+    for (int d = 0; d < a.DR; d += 16)
+      acc = mm_piece<kF32>(*reinterpret_cast<const uint4*>(xp + d),
+                           *reinterpret_cast<const uint4*>(kp + d), acc);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) (wave == 0 ? kk : qk)[4 * g + e][l15] = acc[e];
+  }
+  __syncthreads();
+  const int R = a.H / a.G;
+  for (int h0 = 0; h0 < R; h0 += 16) {
+    // sixteen lanes per head, lane c = column c (and token c)
+    const int hs = wave * 4 + g, hl = h0 + hs, h = gh * R + min(hl, R - 1), c = l15;
+    const bool ok = c < cnt;
+    const float* ab = a.ab + (long long)(n0 + min(c, cnt - 1)) * a.ldab;
+    const float ld = ok ? fmaxf(-expf(a.a_log[h]) * softplus32(ab[h] + a.dt_bias[h]), -1e30f) : 0.f;
+    const float beta = ok ? sigmoid32(ab[a.H + h]) : 0.f;
+    float t[16], p[16];
+    float s = 0.f, pre = 0.f, suf = 0.f, all = 0.f;
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+      const float li = __shfl(ld, 16 * g + i, 64), bi = __shfl(beta, 16 * g + i, 64);
+      all += li;
+      if (i <= c) pre += li;
+      if (i > c) { s += li; suf += li; }
+      const float gi = expf(s);  // decay over tokens c + 1 .. i (1 at i = c)
+      am[hs][i][c] = i > c ? bi * gi * kk[i][c] : 0.f;
+      p[i] = i >= c ? gi * qk[i][c] : 0.f;
+    }
+    __builtin_amdgcn_wave_barrier();  // each head's matrix is one wave's own
+    // column c of (I + A)^-1 by forward substitution
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+      float v = i == c ? 1.f : 0.f;
+#pragma unroll
+      for (int j = 0; j < i; ++j) v = fmaf(-am[hs][i][j], t[j], v);
+      t[i] = v;
+    }
+    if (hl < R) {
+      float* tp = a.tp + ((long long)ch * a.H + h) * 512 + c;
+#pragma unroll
+      for (int i = 0; i < 16; ++i) { tp[16 * i] = t[i]; tp[256 + 16 * i] = p[i]; }
+      *reinterpret_cast<float4*>(a.gm + (((long long)ch * a.H + h) * 16 + c) * 4) =
+          make_float4(expf(pre), beta, expf(suf), expf(all));
+    }
+    __builtin_amdgcn_wave_barrier();
+  }
+}
 
-// grid (ceil(vdim / 16), H, B), 256 threads: wave w = columns 4w..4w+3, 16 lanes per column;
-// lane lr holds rows 64 i + 4 lr + {0..3}, i < NI (dim <= 64 NI)
+// grid (ceil(vdim / 16), H, B), 256 threads; wave w: rows [16 NI w, 16 NI (w + 1)), DR = 64 NI
 template <int DT, int NI>
 __global__ __launch_bounds__(256) void mixer_delta_scan_kernel(DeltaArgs a) {
   using E = typename St<DT>::E;
   constexpr int DR = 64 * NI;
-  __shared__ __attribute__((aligned(16))) float ks[2][kScanTok][DR], qs[2][kScanTok][DR];
-  __shared__ float vs[2][kScanTok][16], sc[2][kScanTok][4];  // sc: decay, beta, q.k
+  __shared__ __attribute__((aligned(16))) float ex[2][4][2][64][4];
   const SeqRow sq = a.seq[blockIdx.z];
   const int h = blockIdx.y, R = a.H / a.G, gh = h / R, c0 = blockIdx.x * 16;
-  const int tid = threadIdx.x, lane = tid & 63, lr = lane & 15;
-  const int cl = (tid >> 6) * 4 + (lane >> 4), col = c0 + cl;
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, l15 = lane & 15, g = lane >> 4;
+  const int col = c0 + l15;
   const bool cok = col < a.vdim;
+  const int r0 = 16 * NI * wave;
   float* st = a.state + sq.slot * a.s_slot + (long long)h * a.dim * a.EP;
-  float S[NI][4];
+  cf32x4 S[NI];
 #pragma unroll
   for (int i = 0; i < NI; ++i)
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
-      const int r = 64 * i + 4 * lr + e;
+      const int r = r0 + 16 * i + 4 * g + e;
       S[i][e] = sq.pos0 > 0 && cok && r < a.dim ? st[(long long)r * a.EP + col] : 0.f;
     }
-  // staging: thread -> (token tid / 16, 16 lanes over the row), pieces in registers
-  const int tt = tid >> 4, tl = tid & 15;
-  float pk[4 * NI], pq[4 * NI], pv, ps;
-  auto gload = [&](int t0) __attribute__((always_inline)) {
-    const int t = min(t0 + tt, sq.len - 1);  // rows past the end repeat the last (not used)
-    const long long n = sq.row0 + t;
-    const float* kp = a.kn + (n * a.G + gh) * a.dim;
-    const float* qp = a.qn + (n * a.G + gh) * a.dim;
+  const int nc = (sq.len + kChunk - 1) / kChunk, ch0 = a.chunk0[blockIdx.z];
+  const long long last = sq.row0 + sq.len - 1;
+
+  // one chunk's operands; rows past the end repeat the last (their beta is zero)
+  uint4 kp[NI], qp[NI], tq, pq;
+  float kt[NI][4], vv[4];
+  float4 gm[4];
+  auto load = [&](int c) __attribute__((always_inline)) {
+    const long long n = (long long)sq.row0 + kChunk * c;
+    const long long nr = min(n + l15, last);
+    const float* kr = a.kn + (nr * a.G + gh) * DR + r0 + 4 * g;
+    const float* qr = a.qn + (nr * a.G + gh) * DR + r0 + 4 * g;
 #pragma unroll
-    for (int i = 0; i < 4 * NI; ++i) {
-      const int d = tl + 16 * i;
-      pk[i] = d < a.dim ? kp[d] : 0.f;
-      pq[i] = d < a.dim ? qp[d] : 0.f;
+    for (int i = 0; i < NI; ++i) {
+      kp[i] = *reinterpret_cast<const uint4*>(kr + 16 * i);
+      qp[i] = *reinterpret_cast<const uint4*>(qr + 16 * i);
     }
-    pv = c0 + tl < a.vdim ? a.vv[(n * a.H + h) * a.vdim + c0 + tl] : 0.f;
-    ps = tl < 2 ? a.bd[(n * a.H + h) * 2 + tl] : tl == 2 ? a.qk[n * a.G + gh] : 0.f;
+    const float* tp = a.tp + ((long long)(ch0 + c) * a.H + h) * 512 + 16 * l15 + 4 * g;
+    tq = *reinterpret_cast<const uint4*>(tp);
+    pq = *reinterpret_cast<const uint4*>(tp + 256);
+    const float4* gp = reinterpret_cast<const float4*>(a.gm) +
+                       ((long long)(ch0 + c) * a.H + h) * 16 + 4 * g;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const long long nt = min(n + 4 * g + e, last);
+      gm[e] = gp[e];
+      vv[e] = cok ? a.vv[(nt * a.H + h) * a.vdim + col] : 0.f;
+#pragma unroll
+      for (int i = 0; i < NI; ++i) kt[i][e] = a.kn[(nt * a.G + gh) * DR + r0 + 16 * i + l15];
+    }
   };
-  auto sstore = [&](int buf) __attribute__((always_inline)) {
+  load(0);
+  for (int c = 0; c < nc; ++c) {
+    const int buf = c & 1;
+    cf32x4 ks{0.f, 0.f, 0.f, 0.f}, qs{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int i = 0; i < 4 * NI; ++i) {
-      ks[buf][tt][tl + 16 * i] = pk[i];
-      qs[buf][tt][tl + 16 * i] = pq[i];
+    for (int i = 0; i < NI; ++i) {
+      const uint4 sb = __builtin_bit_cast(uint4, S[i]);
+      ks = mm_piece<kF32>(kp[i], sb, ks);
+      qs = mm_piece<kF32>(qp[i], sb, qs);
     }
-    vs[buf][tt][tl] = pv;
-    if (tl < 4) sc[buf][tt][tl] = ps;
-  };
-  gload(0);
-  sstore(0);
-  __syncthreads();
-  int buf = 0;
-  for (int t0 = 0; t0 < sq.len; t0 += kScanTok) {
-    const bool more = t0 + kScanTok < sq.len;
-    if (more) gload(t0 + kScanTok);
-    const int nt = min(kScanTok, sq.len - t0);
-    float oreg = 0.f;
-#pragma unroll 4
-    for (int t = 0; t < nt; ++t) {
-      float4 kv[NI], qv[NI];
+    *reinterpret_cast<cf32x4*>(ex[buf][wave][0][lane]) = ks;
+    *reinterpret_cast<cf32x4*>(ex[buf][wave][1][lane]) = qs;
+    const uint4 tc = tq, pc = pq;
+    float ktc[NI][4], vc[4];
+    float4 gc[4];
 #pragma unroll
-      for (int i = 0; i < NI; ++i) {
-        kv[i] = *reinterpret_cast<const float4*>(&ks[buf][t][64 * i + 4 * lr]);
-        qv[i] = *reinterpret_cast<const float4*>(&qs[buf][t][64 * i + 4 * lr]);
-      }
-      const float dec = sc[buf][t][0], beta = sc[buf][t][1], qk = sc[buf][t][2];
-      const float v = vs[buf][t][cl];
-      float ka = 0.f, kb = 0.f, qa = 0.f, qb = 0.f;
+    for (int e = 0; e < 4; ++e) {
+      gc[e] = gm[e];
+      vc[e] = vv[e];
 #pragma unroll
-      for (int i = 0; i < NI; ++i) {
-        ka = fmaf(kv[i].x, S[i][0], ka); kb = fmaf(kv[i].y, S[i][1], kb);
-        qa = fmaf(qv[i].x, S[i][0], qa); qb = fmaf(qv[i].y, S[i][1], qb);
-        ka = fmaf(kv[i].z, S[i][2], ka); kb = fmaf(kv[i].w, S[i][3], kb);
-        qa = fmaf(qv[i].z, S[i][2], qa); qb = fmaf(qv[i].w, S[i][3], qb);
-      }
-      const float kS = row16_sum(ka + kb), qS = row16_sum(qa + qb);
-      const float u = beta * (v - dec * kS);
-#pragma unroll
-      for (int i = 0; i < NI; ++i) {
-        S[i][0] = fmaf(kv[i].x, u, dec * S[i][0]);
-        S[i][1] = fmaf(kv[i].y, u, dec * S[i][1]);
-        S[i][2] = fmaf(kv[i].z, u, dec * S[i][2]);
-        S[i][3] = fmaf(kv[i].w, u, dec * S[i][3]);
-      }
-      const float ov = fmaf(dec, qS, qk * u);
-      oreg = lr == t ? ov : oreg;  // lane lr keeps token lr of the round
+      for (int i = 0; i < NI; ++i) ktc[i][e] = kt[i][e];
     }
-    if (cok && lr < nt)
-      a.o[((long long)(sq.row0 + t0 + lr) * a.H + h) * a.vdim + col] = oreg;
-    if (more) sstore(buf ^ 1);
+    if (c + 1 < nc) load(c + 1);
     __syncthreads();
-    buf ^= 1;
+    ks = *reinterpret_cast<const cf32x4*>(ex[buf][0][0][lane]);
+#pragma unroll
+    for (int w = 1; w < 4; ++w) ks += *reinterpret_cast<const cf32x4*>(ex[buf][w][0][lane]);
+    cf32x4 rhs;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) rhs[e] = gc[e].y * (vc[e] - gc[e].x * ks[e]);
+    const cf32x4 u = mm_piece<kF32>(tc, __builtin_bit_cast(uint4, rhs), cf32x4{0.f, 0.f, 0.f, 0.f});
+    cf32x4 ud;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) ud[e] = gc[e].z * u[e];
+    const uint4 ub = __builtin_bit_cast(uint4, ud);
+#pragma unroll
+    for (int i = 0; i < NI; ++i) {
+      const cf32x4 ka = {ktc[i][0], ktc[i][1], ktc[i][2], ktc[i][3]};
+      S[i] = mm_piece<kF32>(__builtin_bit_cast(uint4, ka), ub, S[i] * gc[0].w);
+    }
+    if (wave == (c & 3)) {  // the read-outs of a chunk: the waves take turns
+      qs = *reinterpret_cast<const cf32x4*>(ex[buf][0][1][lane]);
+#pragma unroll
+      for (int w = 1; w < 4; ++w) qs += *reinterpret_cast<const cf32x4*>(ex[buf][w][1][lane]);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) qs[e] *= gc[e].x;
+      const cf32x4 o = mm_piece<kF32>(pc, __builtin_bit_cast(uint4, u), qs);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const int t = kChunk * c + 4 * g + e;
+        if (cok && t < sq.len) a.o[((long long)(sq.row0 + t) * a.H + h) * a.vdim + col] = o[e];
+      }
+    }
   }
   if (cok)
 #pragma unroll
     for (int i = 0; i < NI; ++i)
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
-        const int r = 64 * i + 4 * lr + e;
+        const int r = r0 + 16 * i + 4 * g + e;
         if (r < a.dim) st[(long long)r * a.EP + col] = S[i][e];
       }
   // the ring entries of the last taps - 1 tokens (every prompt row has been convolved by now)
@@ -234,11 +343,11 @@ __global__ __launch_bounds__(256) void mixer_delta_scan_kernel(DeltaArgs a) {
   const int nq = h % R == 0 ? 2 * a.dim : 0;  // q and k channels: the group's first head
   for (int i = tid; i < keep * (nq + a.vdim); i += 256) {
     const int j = i / (nq + a.vdim), x = i - j * (nq + a.vdim);
-    const int c = x < nq ? (x < a.dim ? gh * a.dim + x : (a.G + gh) * a.dim + x - a.dim)
-                         : 2 * a.G * a.dim + h * a.vdim + x - nq;
+    const int cc = x < nq ? (x < a.dim ? gh * a.dim + x : (a.G + gh) * a.dim + x - a.dim)
+                          : 2 * a.G * a.dim + h * a.vdim + x - nq;
     const int row = sq.len - 1 - j;
-    ring[(long long)((sq.pos0 + row) % a.taps) * C + c] =
-        St<DT>::ld(reinterpret_cast<const E*>(a.proj)[(long long)(sq.row0 + row) * a.ldp + c]);
+    ring[(long long)((sq.pos0 + row) % a.taps) * C + cc] =
+        St<DT>::ld(reinterpret_cast<const E*>(a.proj)[(long long)(sq.row0 + row) * a.ldp + cc]);
   }
 }
 
@@ -252,6 +361,34 @@ __global__ __launch_bounds__(256) void mixer_delta_out_kernel(DeltaArgs a) {
   const long long n = item / a.H;
   const int h = (int)(item - n * a.H);
   const float* o = a.o + item * a.vdim;
+  E* out = reinterpret_cast<E*>(a.out) + n * a.ldo + h * a.vdim;
+  const E* gp = reinterpret_cast<const E*>(a.proj) + n * a.ldp + delta_channels(a) + h * a.vdim;
+  if constexpr (DT != kF32) {
+    // two consecutive channels per lane and access where rows allow it
+    if (a.vdim % 2 == 0 && a.ldp % 2 == 0 && a.ldo % 2 == 0 && delta_channels(a) % 2 == 0) {
+      float2 x[2];
+      float ss = 0.f;
+#pragma unroll
+      for (int i = 0; i < 2; ++i) {
+        const int d = 2 * lane + 128 * i;
+        x[i] = d < a.vdim ? *reinterpret_cast<const float2*>(o + d) : make_float2(0.f, 0.f);
+        ss += x[i].x * x[i].x + x[i].y * x[i].y;
+      }
+      const float r = 1.f / sqrtf(wave_sum(ss) / (float)a.vdim + a.eps);
+#pragma unroll
+      for (int i = 0; i < 2; ++i) {
+        const int d = 2 * lane + 128 * i;
+        if (d >= a.vdim) continue;
+        const uint32_t z = *reinterpret_cast<const uint32_t*>(gp + d);
+        const float2 w = *reinterpret_cast<const float2*>(a.norm_w + d);
+        const float y0 = x[i].x * r * w.x * silu32(St<DT>::ld((uint16_t)(z & 0xffffu)));
+        const float y1 = x[i].y * r * w.y * silu32(St<DT>::ld((uint16_t)(z >> 16)));
+        *reinterpret_cast<uint32_t*>(out + d) =
+            (uint32_t)St<DT>::st(y0) | ((uint32_t)St<DT>::st(y1) << 16);
+      }
+      return;
+    }
+  }
   float x[4], ss = 0.f;
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
@@ -260,8 +397,6 @@ __global__ __launch_bounds__(256) void mixer_delta_out_kernel(DeltaArgs a) {
     ss += x[i] * x[i];
   }
   const float r = 1.f / sqrtf(wave_sum(ss) / (float)a.vdim + a.eps);
-  const E* gp = reinterpret_cast<const E*>(a.proj) + n * a.ldp + delta_channels(a) + h * a.vdim;
-  E* out = reinterpret_cast<E*>(a.out) + n * a.ldo + h * a.vdim;
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
     const int d = lane + 64 * i;
@@ -389,21 +524,27 @@ CAKE_API int cake_mixer_delta_prefill(int dt, const void* proj, long long ldp, c
                                       int EP, int taps, float eps, const float* conv,
                                       const float* a_log, const float* dt_bias,
                                       const float* norm_w, float* qn, float* kn, float* vv,
-                                      float* qk, float* bd, float* o, float* state, float* ring,
+                                      float* tp, float* gm, float* o, float* state, float* ring,
                                       long long s_slot, long long r_slot, const int* row_pos,
                                       const int* row_slot, const int* row_seq0, const void* seq,
-                                      int B, void* out, long long ldo, hipStream_t st) {
-  if (!delta_shape_ok(H, G, dim, vdim, EP, taps) || N <= 0 || B <= 0)
+                                      int B, const void* chunk, const int* chunk0, int NC,
+                                      void* out, long long ldo, hipStream_t st) {
+  if (!delta_shape_ok(H, G, dim, vdim, EP, taps) || N <= 0 || B <= 0 || NC < B)
     return (int)hipErrorInvalidValue;
+  const int ni = (dim + 63) / 64;
   DeltaArgs a{proj, ldp, ab, ldab, N, H, G, dim, vdim, EP, taps, eps, conv, a_log, dt_bias,
-              norm_w, qn, kn, vv, qk, bd, o, state, ring, s_slot, r_slot, row_pos, row_slot,
-              row_seq0, (const SeqRow*)seq, out, ldo};
-  const dim3 gp((unsigned)(((long long)N * (G + H) + 3) / 4));
+              norm_w, 64 * ni, qn, kn, vv, tp, gm, o, state, ring, s_slot, r_slot, row_pos,
+              row_slot, row_seq0, (const SeqRow*)seq, (const int2*)chunk, chunk0, NC, out, ldo};
+  const dim3 gp((unsigned)(((long long)NC * (2 * G + H) + 3) / 4));
   const dim3 gs((vdim + 15) / 16, H, B);
   const dim3 go((unsigned)(((long long)N * H + 3) / 4));
-  const int ni = (dim + 63) / 64;
+  const int widest = 64 * ni > vdim ? 64 * ni : vdim;
+  const int vec = dim % 2 == 0 && vdim % 2 == 0 && ldp % 2 == 0 && ((uintptr_t)proj % 4) == 0;
   CAKE_MIX_DT(dt, {
-    hipLaunchKernelGGL((mixer_delta_prep_kernel<DT>), gp, dim3(256), 0, st, a);
+    if (widest <= 64) hipLaunchKernelGGL((mixer_delta_prep_kernel<DT, 1>), gp, dim3(256), 0, st, a, vec);
+    else if (widest <= 128) hipLaunchKernelGGL((mixer_delta_prep_kernel<DT, 2>), gp, dim3(256), 0, st, a, vec);
+    else hipLaunchKernelGGL((mixer_delta_prep_kernel<DT, 4>), gp, dim3(256), 0, st, a, vec);
+    hipLaunchKernelGGL(mixer_delta_chunk_kernel, dim3(NC, G), dim3(256), 0, st, a);
     if (ni == 1) hipLaunchKernelGGL((mixer_delta_scan_kernel<DT, 1>), gs, dim3(256), 0, st, a);
     else if (ni == 2) hipLaunchKernelGGL((mixer_delta_scan_kernel<DT, 2>), gs, dim3(256), 0, st, a);
     else if (ni == 3) hipLaunchKernelGGL((mixer_delta_scan_kernel<DT, 3>), gs, dim3(256), 0, st, a);

@@ -98,8 +98,16 @@ __global__ __launch_bounds__(kGemvThreads) void mixer_loop_kernel(
   const uint16_t *wa0, *wb0;
   map(p0 < npairs ? p0 : npairs - 1, wa0, wb0);
   if (PFC > 0 && p0 < npairs) prefetch_rows<PFC>(wa0, wb0, pre);
-  for (int i = threadIdx.x; i < K; i += kGemvThreads)
-    xs[i] = i < W ? x[i] : i < 2 * W ? x0[i - W] : 0.f;
+  if (W % 4 == 0) {
+    for (int i = threadIdx.x * 4; i < K; i += kGemvThreads * 4)
+      *reinterpret_cast<float4*>(xs + i) =
+          i < W ? *reinterpret_cast<const float4*>(x + i)
+                : i < 2 * W ? *reinterpret_cast<const float4*>(x0 + i - W)
+                            : make_float4(0.f, 0.f, 0.f, 0.f);
+  } else {
+    for (int i = threadIdx.x; i < K; i += kGemvThreads)
+      xs[i] = i < W ? x[i] : i < 2 * W ? x0[i - W] : 0.f;
+  }
   __syncthreads();
   auto epi = [&](int p, float da, float db) {
     if (lane > 1) return;

@@ -11,10 +11,17 @@ __global__ __launch_bounds__(256) void mixer_embed_kernel(const void* table, con
   using E = typename St<DT>::E;
   const E* row = reinterpret_cast<const E*>(table) + (long long)tok[blockIdx.x] * ld;
   const long long o = (long long)blockIdx.x * ld;
-  for (int i = threadIdx.x; i < ld; i += 256) {
-    const float v = St<DT>::ld(row[i]);
-    x[o + i] = v;
-    if (x0) x0[o + i] = v;
+  for (int i = threadIdx.x * 4; i < ld; i += 1024) {  // ld % 8 == 0
+    float4 v;
+    if constexpr (DT == kF32) {
+      v = *reinterpret_cast<const float4*>(row + i);
+    } else {
+      const uint2 w = *reinterpret_cast<const uint2*>(row + i);
+      v = make_float4(St<DT>::ld((uint16_t)(w.x & 0xffffu)), St<DT>::ld((uint16_t)(w.x >> 16)),
+                      St<DT>::ld((uint16_t)(w.y & 0xffffu)), St<DT>::ld((uint16_t)(w.y >> 16)));
+    }
+    *reinterpret_cast<float4*>(x + o + i) = v;
+    if (x0) *reinterpret_cast<float4*>(x0 + o + i) = v;
   }
 }
 
@@ -67,6 +74,20 @@ __global__ __launch_bounds__(256) void mixer_loop_rows_kernel(const float* x, co
   using E = typename St<DT>::E;
   const long long n = blockIdx.x;
   E* o = reinterpret_cast<E*>(a) + n * lda;
+  if (DT != kF32 && W % 8 == 0 && lda % 4 == 0) {
+    for (int i = threadIdx.x * 4; i < lda; i += 1024) {
+      const float4 v = i < W ? *reinterpret_cast<const float4*>(x + n * ldx + i)
+                       : i < 2 * W ? *reinterpret_cast<const float4*>(x0 + n * ldx + i - W)
+                                   : make_float4(0.f, 0.f, 0.f, 0.f);
+      *reinterpret_cast<uint2*>(o + i) =
+          make_uint2((uint32_t)St<DT>::st(v.x) | ((uint32_t)St<DT>::st(v.y) << 16),
+                     (uint32_t)St<DT>::st(v.z) | ((uint32_t)St<DT>::st(v.w) << 16));
+    }
+    for (int i = threadIdx.x * 4; i < ldx; i += 1024)
+      *reinterpret_cast<float4*>(y + n * ldx + i) =
+          i < W ? *reinterpret_cast<const float4*>(step + i) : make_float4(0.f, 0.f, 0.f, 0.f);
+    return;
+  }
   for (int i = threadIdx.x; i < lda; i += 256)
     o[i] = St<DT>::st(i < W ? x[n * ldx + i] : i < 2 * W ? x0[n * ldx + i - W] : 0.f);
   for (int i = threadIdx.x; i < ldx; i += 256) y[n * ldx + i] = i < W ? step[i] : 0.f;
@@ -90,7 +111,7 @@ using namespace cake;
 
 CAKE_API int cake_mixer_embed(int dt, const void* table, const int* tok, int N, int ld, float* x,
                               float* x0, hipStream_t st) {
-  if (N < 0 || ld <= 0) return (int)hipErrorInvalidValue;
+  if (N < 0 || ld <= 0 || ld % 8) return (int)hipErrorInvalidValue;
   if (N == 0) return 0;
   CAKE_MIX_DT(dt, hipLaunchKernelGGL((mixer_embed_kernel<DT>), dim3(N), dim3(256), 0, st, table,
                                      tok, ld, x, x0));

@@ -204,7 +204,7 @@ _LIB_SIGS = {
         "cake_mixer_attn_decode": [I, P, L, I, P, P, P, I, I, I, I, F, F, P, P, L, L, P, L, I, I,
                                    I, I, I, I, I, I, P, P, P],
         "cake_mixer_delta_prefill": [I, P, L, P, L, I, I, I, I, I, I, I, F, P, P, P, P, P, P, P,
-                                     P, P, P, P, P, L, L, P, P, P, P, I, P, L, P],
+                                     P, P, P, P, P, L, L, P, P, P, P, I, P, P, I, P, L, P],
         "cake_mixer_delta_decode": [I, P, L, P, L, I, I, I, I, I, I, I, F, P, P, P, P, P, P, L, L,
                                     P, P, P, L, P],
     },

@@ -15,6 +15,7 @@ from ._lib import check, library
 
 DT = {torch.bfloat16: 0, torch.float16: 1, torch.float32: 2}
 MAX_HEAD = 256   # largest head size the kernels hold
+CHUNK = 16       # tokens of one delta-rule chunk
 MAX_SPLIT = 64   # key splits of one decode-attention launch
 
 
@@ -58,6 +59,8 @@ class Rows:
     slot: torch.Tensor   # [N]
     first: torch.Tensor  # [N] packed row of the sequence's first token of this step
     seq: torch.Tensor    # [B, 4]: first row, length, first position, slot
+    chunk: torch.Tensor  # [NC, 2]: the sequences cut into runs of CHUNK tokens (first row, tokens)
+    chunk0: torch.Tensor  # [B] first chunk of each sequence
     host: list           # [(first row, length, first position, slot)]
 
     @classmethod
@@ -74,10 +77,21 @@ class Rows:
             slot += [s] * n
             first += [r0] * n
         N, B = len(tok), len(host)
-        flat = torch.tensor(tok + pos + slot + first + [x for h in host for x in h],
-                            dtype=torch.int32).to(device)
-        t = [flat[i * N:(i + 1) * N] for i in range(4)]
-        return cls(N, B, max(h[1] for h in host), *t, flat[4 * N:].view(B, 4), host)
+        chunks, chunk0 = [], []
+        for r0, n, _, _ in host:
+            chunk0.append(len(chunks))
+            chunks += [(r0 + c, min(CHUNK, n - c)) for c in range(0, n, CHUNK)]
+        parts = [tok, pos, slot, first, chunk0, [x for h in host for x in h],
+                 [x for c in chunks for x in c]]
+        # every part starts on 16 bytes (the kernels read rows of seq and chunk whole)
+        flat, at = [], []
+        for p in parts:
+            at.append(len(flat))
+            flat += p + [0] * (-len(p) % 4)
+        flat = torch.tensor(flat, dtype=torch.int32).to(device)
+        tok, pos, slot, first, chunk0, seq, chunk = (flat[a:a + len(p)] for a, p in zip(at, parts))
+        return cls(N, B, max(h[1] for h in host), tok, pos, slot, first, seq.view(B, 4),
+                   chunk.view(-1, 2), chunk0, host)
 
 
 def embed(table, tok, x, x0=None):
@@ -323,8 +337,8 @@ def delta_prompt(sh: DeltaShape, proj, ab, rows: Rows, eps: float, conv, a_log, 
     pp, ldp = _mat(proj, "proj", proj.dtype, N, sh.channels + sh.out_cols)
     abp, ldab = _mat(ab, "ab", f, N, 2 * sh.heads)
     op, ldo = _mat(out, "out", proj.dtype, N, sh.out_cols)
-    G, H = sh.kv_heads, sh.heads
-    sizes = (N * G * sh.dim, N * G * sh.dim, N * H * sh.vdim, N * G, 2 * N * H, N * H * sh.vdim)
+    G, H, NC, DR = sh.kv_heads, sh.heads, rows.chunk.shape[0], pad_to(sh.dim, 64)
+    sizes = (N * G * DR, N * G * DR, N * H * sh.vdim, NC * H * 512, NC * H * 64, N * H * sh.vdim)
     ws = torch.empty(sum(pad_to(s, 4) for s in sizes), device=dev, dtype=f)
     ptrs, o = [], 0
     for s in sizes:
@@ -335,7 +349,8 @@ def delta_prompt(sh: DeltaShape, proj, ab, rows: Rows, eps: float, conv, a_log, 
         DT[proj.dtype], pp, ldp, abp, ldab, N, H, G, sh.dim, sh.vdim, sh.EP, sh.taps, float(eps),
         *_delta_consts(sh, conv, a_log, dt_bias, norm_w), *ptrs, sp, rp, s_slot, r_slot,
         rows.pos.data_ptr(), rows.slot.data_ptr(), rows.first.data_ptr(), rows.seq.data_ptr(),
-        rows.B, op, ldo, _stream()), "mixer_delta_prefill")
+        rows.B, rows.chunk.data_ptr(), rows.chunk0.data_ptr(), NC, op, ldo, _stream()),
+        "mixer_delta_prefill")
 
 
 def delta_decode(sh: DeltaShape, proj, ab, pos, slot, eps: float, conv, a_log, dt_bias, norm_w,

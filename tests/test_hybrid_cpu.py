@@ -177,6 +177,10 @@ def test_rows_pack():
     assert r.tok.tolist() == [5, 6, 7, 9] and r.pos.tolist() == [0, 1, 2, 10]
     assert r.slot.tolist() == [3, 3, 3, 1] and r.first.tolist() == [0, 0, 0, 3]
     assert r.seq.tolist() == [[0, 3, 0, 3], [3, 1, 10, 1]]
+    r = Rows.pack([(0, 0, [1] * 33), (1, 0, [1] * 16), (2, 5, [1])], "cpu")
+    assert r.chunk.tolist() == [[0, 16], [16, 16], [32, 1], [33, 16], [49, 1]]
+    assert r.chunk0.tolist() == [0, 3, 4]
+    assert all(t.data_ptr() % 16 == 0 for t in (r.seq, r.chunk))
     with pytest.raises(ValueError):
         Rows.pack([(0, 0, [])], "cpu")
 
