@@ -37,56 +37,74 @@ struct PrepArgs {
   long long k_slot, v_slot;  // elements per slot
 };
 
-// LPH lanes per (row, head), four consecutive dims each
-template <int DT>
-__global__ __launch_bounds__(256) void mixer_prep_qk_kernel(PrepArgs a, int lph, int vec) {
+// sum over aligned groups of `lph` lanes (a power of two): DPP inside 16-lane rows, lane swaps
+// across them
+__device__ __forceinline__ float lanes_sum(float v, int lph) {
+  if (lph >= 2) v += dpp_f<kDppXor1>(v);
+  if (lph >= 4) v += dpp_f<kDppXor2>(v);
+  if (lph >= 8) v += dpp_f<kDppHalfMirror>(v);
+  if (lph >= 16) v += dpp_f<kDppMirror>(v);
+  if (lph >= 32) v = xor_add<16>(v);
+  if (lph >= 64) v = xor_add<32>(v);
+  return v;
+}
+
+// lph lanes per (row, head), EPL consecutive dims each.  VEC: rows and heads on 2 EPL-byte
+// boundaries and dim % EPL == 0 (16-bit types).
+template <int DT, int EPL, bool VEC>
+__global__ __launch_bounds__(256) void mixer_prep_qk_kernel(PrepArgs a, int lph) {
   using E = typename St<DT>::E;
   const int per = 256 / lph;  // (row, head) items per workgroup
   const int item = blockIdx.x * per + threadIdx.x / lph;
-  const int l = threadIdx.x % lph, d0 = 4 * l;
+  const int l = threadIdx.x % lph, d0 = EPL * l;
   const int nh = a.H + a.G;
-  if (item >= a.N * nh) return;  // whole lph-lane groups leave together
-  const int n = item / nh, hh = item - n * nh;
+  const bool live = item < a.N * nh;  // lanes past the end shadow the last item
+  const int it = live ? item : a.N * nh - 1;
+  const int n = it / nh, hh = it - n * nh;
   const bool isq = hh < a.H;
   const int pos = a.row_pos[n];
   const E* src = reinterpret_cast<const E*>(a.proj) + (long long)n * a.ldp + (long long)hh * a.dim;
-  float x[4];
-  if (DT != kF32 && vec) {  // rows and heads on 8-byte boundaries, dim % 4 == 0
-    const uint2 w = d0 < a.dim ? *reinterpret_cast<const uint2*>(src + d0) : make_uint2(0u, 0u);
-    x[0] = St<DT>::ld((uint16_t)(w.x & 0xffffu)); x[1] = St<DT>::ld((uint16_t)(w.x >> 16));
-    x[2] = St<DT>::ld((uint16_t)(w.y & 0xffffu)); x[3] = St<DT>::ld((uint16_t)(w.y >> 16));
+  float x[EPL];
+  if constexpr (VEC && EPL == 8) {
+    unpack8<DT == kF32 ? kBF16 : DT>(d0 < a.dim ? *reinterpret_cast<const uint4*>(src + d0)
+                                                : make_uint4(0u, 0u, 0u, 0u), x);
   } else {
 #pragma unroll
-    for (int e = 0; e < 4; ++e) x[e] = d0 + e < a.dim ? St<DT>::ld(src[d0 + e]) : 0.f;
+    for (int e = 0; e < EPL; ++e) x[e] = d0 + e < a.dim ? St<DT>::ld(src[d0 + e]) : 0.f;
   }
+  const float2* cs = a.cs + (long long)pos * a.rd2;
 #pragma unroll
-  for (int p = 0; p < 2; ++p) {
-    const int i = 2 * l + p;
+  for (int p = 0; p < EPL / 2; ++p) {
+    const int i = EPL / 2 * l + p;
     if (i < a.rd2) {
-      const float2 t = a.cs[(long long)pos * a.rd2 + i];
+      const float2 t = cs[i];
       const float u = x[2 * p], v = x[2 * p + 1];
       x[2 * p] = u * t.x - v * t.y;
       x[2 * p + 1] = v * t.x + u * t.y;
     }
   }
   if (a.qk_norm) {
-    float ss = x[0] * x[0] + x[1] * x[1] + x[2] * x[2] + x[3] * x[3];
-    for (int o = lph >> 1; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
-    const float r = 1.f / sqrtf(ss / (float)a.dim + a.eps);
+    float ss = 0.f;
 #pragma unroll
-    for (int e = 0; e < 4; ++e) x[e] *= r;
+    for (int e = 0; e < EPL; ++e) ss += x[e] * x[e];
+    const float r = 1.f / sqrtf(lanes_sum(ss, lph) / (float)a.dim + a.eps);
+#pragma unroll
+    for (int e = 0; e < EPL; ++e) x[e] *= r;
   }
   E* dst = isq ? reinterpret_cast<E*>(a.qn) + ((long long)n * a.H + hh) * a.DP
                : reinterpret_cast<E*>(a.kc) + a.row_slot[n] * a.k_slot +
                      ((long long)(hh - a.H) * a.S + pos) * a.DP;
-  if (d0 < a.DP) {  // DP % 4 == 0; columns past dim carry zeros
-    if constexpr (DT == kF32) {
-      *reinterpret_cast<float4*>(dst + d0) = make_float4(x[0], x[1], x[2], x[3]);
-    } else {
-      const uint32_t lo = (uint32_t)St<DT>::st(x[0]) | ((uint32_t)St<DT>::st(x[1]) << 16);
-      const uint32_t hi = (uint32_t)St<DT>::st(x[2]) | ((uint32_t)St<DT>::st(x[3]) << 16);
-      *reinterpret_cast<uint2*>(dst + d0) = make_uint2(lo, hi);
-    }
+  if (!live || d0 >= a.DP) return;  // DP % 8 == 0; columns past dim carry zeros
+  if constexpr (DT == kF32) {
+#pragma unroll
+    for (int e = 0; e < EPL; e += 4)
+      *reinterpret_cast<float4*>(dst + d0 + e) = make_float4(x[e], x[e + 1], x[e + 2], x[e + 3]);
+  } else {
+    uint32_t w[EPL / 2];
+#pragma unroll
+    for (int e = 0; e < EPL / 2; ++e)
+      w[e] = (uint32_t)St<DT>::st(x[2 * e]) | ((uint32_t)St<DT>::st(x[2 * e + 1]) << 16);
+    *reinterpret_cast<uint4*>(dst + d0) = make_uint4(w[0], w[1], w[2], w[3]);
   }
 }
 
@@ -655,14 +673,17 @@ CAKE_API int cake_mixer_prep(int dt, const void* proj, long long ldp, int N, int
   if (N == 0) return 0;
   PrepArgs a{proj, ldp, N, H, G, dim, vdim, DP, DVP, S, rd2, qk_norm, eps, (const float2*)cs,
              row_pos, row_slot, qn, kc, vc, k_slot, v_slot};
-  int lph = 8;
-  while (4 * lph < DP) lph <<= 1;  // <= 64
-  const int vec = dim % 4 == 0 && ldp % 4 == 0 && ((uintptr_t)proj % 8) == 0;
+  int lph = 4;
+  while (8 * lph < DP) lph <<= 1;  // <= 32
+  const bool vec = dt != kF32 && dim % 8 == 0 && ldp % 8 == 0 && ((uintptr_t)proj % 16) == 0;
   const long long items = (long long)N * (H + G);
   const dim3 g1((unsigned)((items + 256 / lph - 1) / (256 / lph)));
   const dim3 g2((N + 63) / 64, (G * ((vdim + 7) / 8) + 3) / 4);
-  CAKE_MIX_DT(dt, hipLaunchKernelGGL((mixer_prep_qk_kernel<DT>), g1, dim3(256), 0, st, a, lph, vec);
-              hipLaunchKernelGGL((mixer_prep_v_kernel<DT>), g2, dim3(256), 0, st, a));
+  CAKE_MIX_DT(dt, {
+    if (vec) hipLaunchKernelGGL((mixer_prep_qk_kernel<DT, 8, true>), g1, dim3(256), 0, st, a, lph);
+    else hipLaunchKernelGGL((mixer_prep_qk_kernel<DT, 8, false>), g1, dim3(256), 0, st, a, lph);
+    hipLaunchKernelGGL((mixer_prep_v_kernel<DT>), g2, dim3(256), 0, st, a);
+  });
   return (int)hipGetLastError();
 }
 

@@ -221,14 +221,22 @@ __global__ __launch_bounds__(256) void mixer_delta_chunk_kernel(DeltaArgs a) {
   }
 }
 
-// grid (ceil(vdim / 16), H, B), 256 threads; wave w: rows [16 NI w, 16 NI (w + 1)), DR = 64 NI
+// One chunk's operands of a scan lane.
+template <int NI> struct ScanSet {
+  u32x4 kp[NI], qp[NI], t, p;
+  float kt[NI][4], v[4];
+  cf32x4 gm[4];
+};
+
+// grid (H, ceil(vdim / 16), B) — the column blocks of a head land on one XCD and share its
+// rows in that L2 — 256 threads; wave w: rows [16 NI w, 16 NI (w + 1)), DR = 64 NI
 template <int DT, int NI>
 __global__ __launch_bounds__(256) void mixer_delta_scan_kernel(DeltaArgs a) {
   using E = typename St<DT>::E;
   constexpr int DR = 64 * NI;
   __shared__ __attribute__((aligned(16))) float ex[2][4][2][64][4];
   const SeqRow sq = a.seq[blockIdx.z];
-  const int h = blockIdx.y, R = a.H / a.G, gh = h / R, c0 = blockIdx.x * 16;
+  const int h = blockIdx.x, R = a.H / a.G, gh = h / R, c0 = blockIdx.y * 16;
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, l15 = lane & 15, g = lane >> 4;
   const int col = c0 + l15;
   const bool cok = col < a.vdim;
@@ -243,89 +251,88 @@ __global__ __launch_bounds__(256) void mixer_delta_scan_kernel(DeltaArgs a) {
       S[i][e] = sq.pos0 > 0 && cok && r < a.dim ? st[(long long)r * a.EP + col] : 0.f;
     }
   const int nc = (sq.len + kChunk - 1) / kChunk, ch0 = a.chunk0[blockIdx.z];
-  const long long last = sq.row0 + sq.len - 1;
+  const int last = sq.row0 + sq.len - 1;
+  const int vcol = cok ? col : 0;
 
-  // one chunk's operands; rows past the end repeat the last (their beta is zero)
-  uint4 kp[NI], qp[NI], tq, pq;
-  float kt[NI][4], vv[4];
-  float4 gm[4];
-  auto load = [&](int c) __attribute__((always_inline)) {
-    const long long n = (long long)sq.row0 + kChunk * c;
+  // rows past the end repeat the last (their beta is zero)
+  auto load = [&](ScanSet<NI>& s, int c) __attribute__((always_inline)) {
+    const int n = sq.row0 + kChunk * c;
     const long long nr = min(n + l15, last);
     const float* kr = a.kn + (nr * a.G + gh) * DR + r0 + 4 * g;
     const float* qr = a.qn + (nr * a.G + gh) * DR + r0 + 4 * g;
 #pragma unroll
     for (int i = 0; i < NI; ++i) {
-      kp[i] = *reinterpret_cast<const uint4*>(kr + 16 * i);
-      qp[i] = *reinterpret_cast<const uint4*>(qr + 16 * i);
+      s.kp[i] = *reinterpret_cast<const u32x4*>(kr + 16 * i);
+      s.qp[i] = *reinterpret_cast<const u32x4*>(qr + 16 * i);
     }
     const float* tp = a.tp + ((long long)(ch0 + c) * a.H + h) * 512 + 16 * l15 + 4 * g;
-    tq = *reinterpret_cast<const uint4*>(tp);
-    pq = *reinterpret_cast<const uint4*>(tp + 256);
-    const float4* gp = reinterpret_cast<const float4*>(a.gm) +
-                       ((long long)(ch0 + c) * a.H + h) * 16 + 4 * g;
+    s.t = *reinterpret_cast<const u32x4*>(tp);
+    s.p = *reinterpret_cast<const u32x4*>(tp + 256);
+    const float* gp = a.gm + (((long long)(ch0 + c) * a.H + h) * 16 + 4 * g) * 4;
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
       const long long nt = min(n + 4 * g + e, last);
-      gm[e] = gp[e];
-      vv[e] = cok ? a.vv[(nt * a.H + h) * a.vdim + col] : 0.f;
+      s.gm[e] = *reinterpret_cast<const cf32x4*>(gp + 4 * e);
+      s.v[e] = a.vv[(nt * a.H + h) * a.vdim + vcol];
 #pragma unroll
-      for (int i = 0; i < NI; ++i) kt[i][e] = a.kn[(nt * a.G + gh) * DR + r0 + 16 * i + l15];
+      for (int i = 0; i < NI; ++i) s.kt[i][e] = a.kn[(nt * a.G + gh) * DR + r0 + 16 * i + l15];
     }
   };
-  load(0);
-  for (int c = 0; c < nc; ++c) {
+  auto chunk = [&](const ScanSet<NI>& s, int c) __attribute__((always_inline)) {
     const int buf = c & 1;
     cf32x4 ks{0.f, 0.f, 0.f, 0.f}, qs{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int i = 0; i < NI; ++i) {
       const uint4 sb = __builtin_bit_cast(uint4, S[i]);
-      ks = mm_piece<kF32>(kp[i], sb, ks);
-      qs = mm_piece<kF32>(qp[i], sb, qs);
+      ks = mm_piece<kF32>(__builtin_bit_cast(uint4, s.kp[i]), sb, ks);
+      qs = mm_piece<kF32>(__builtin_bit_cast(uint4, s.qp[i]), sb, qs);
     }
     *reinterpret_cast<cf32x4*>(ex[buf][wave][0][lane]) = ks;
     *reinterpret_cast<cf32x4*>(ex[buf][wave][1][lane]) = qs;
-    const uint4 tc = tq, pc = pq;
-    float ktc[NI][4], vc[4];
-    float4 gc[4];
-#pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      gc[e] = gm[e];
-      vc[e] = vv[e];
-#pragma unroll
-      for (int i = 0; i < NI; ++i) ktc[i][e] = kt[i][e];
-    }
-    if (c + 1 < nc) load(c + 1);
-    __syncthreads();
+    // the other waves' halves only need the LDS writes: a full barrier would also drain the
+    // operand loads in flight
+    asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
     ks = *reinterpret_cast<const cf32x4*>(ex[buf][0][0][lane]);
 #pragma unroll
     for (int w = 1; w < 4; ++w) ks += *reinterpret_cast<const cf32x4*>(ex[buf][w][0][lane]);
     cf32x4 rhs;
 #pragma unroll
-    for (int e = 0; e < 4; ++e) rhs[e] = gc[e].y * (vc[e] - gc[e].x * ks[e]);
-    const cf32x4 u = mm_piece<kF32>(tc, __builtin_bit_cast(uint4, rhs), cf32x4{0.f, 0.f, 0.f, 0.f});
+    for (int e = 0; e < 4; ++e) rhs[e] = s.gm[e][1] * (s.v[e] - s.gm[e][0] * ks[e]);
+    const cf32x4 u = mm_piece<kF32>(__builtin_bit_cast(uint4, s.t), __builtin_bit_cast(uint4, rhs),
+                                    cf32x4{0.f, 0.f, 0.f, 0.f});
     cf32x4 ud;
 #pragma unroll
-    for (int e = 0; e < 4; ++e) ud[e] = gc[e].z * u[e];
+    for (int e = 0; e < 4; ++e) ud[e] = s.gm[e][2] * u[e];
     const uint4 ub = __builtin_bit_cast(uint4, ud);
 #pragma unroll
     for (int i = 0; i < NI; ++i) {
-      const cf32x4 ka = {ktc[i][0], ktc[i][1], ktc[i][2], ktc[i][3]};
-      S[i] = mm_piece<kF32>(__builtin_bit_cast(uint4, ka), ub, S[i] * gc[0].w);
+      const cf32x4 ka = {s.kt[i][0], s.kt[i][1], s.kt[i][2], s.kt[i][3]};
+      S[i] = mm_piece<kF32>(__builtin_bit_cast(uint4, ka), ub, S[i] * s.gm[0][3]);
     }
     if (wave == (c & 3)) {  // the read-outs of a chunk: the waves take turns
       qs = *reinterpret_cast<const cf32x4*>(ex[buf][0][1][lane]);
 #pragma unroll
       for (int w = 1; w < 4; ++w) qs += *reinterpret_cast<const cf32x4*>(ex[buf][w][1][lane]);
 #pragma unroll
-      for (int e = 0; e < 4; ++e) qs[e] *= gc[e].x;
-      const cf32x4 o = mm_piece<kF32>(pc, __builtin_bit_cast(uint4, u), qs);
+      for (int e = 0; e < 4; ++e) qs[e] *= s.gm[e][0];
+      const cf32x4 o = mm_piece<kF32>(__builtin_bit_cast(uint4, s.p), __builtin_bit_cast(uint4, u), qs);
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
         const int t = kChunk * c + 4 * g + e;
         if (cok && t < sq.len) a.o[((long long)(sq.row0 + t) * a.H + h) * a.vdim + col] = o[e];
       }
     }
+  };
+  // operands two chunks ahead (chunks past the end re-read the last one)
+  ScanSet<NI> s0, s1;
+  load(s0, 0);
+  load(s1, min(1, nc - 1));
+  for (int c = 0; c < nc; c += 2) {
+    chunk(s0, c);
+    if (c + 1 >= nc) break;
+    load(s0, min(c + 2, nc - 1));
+    chunk(s1, c + 1);
+    load(s1, min(c + 3, nc - 1));
   }
   if (cok)
 #pragma unroll
@@ -336,7 +343,7 @@ __global__ __launch_bounds__(256) void mixer_delta_scan_kernel(DeltaArgs a) {
         if (r < a.dim) st[(long long)r * a.EP + col] = S[i][e];
       }
   // the ring entries of the last taps - 1 tokens (every prompt row has been convolved by now)
-  if (blockIdx.x != 0) return;
+  if (blockIdx.y != 0) return;
   const int C = delta_channels(a);
   float* ring = a.ring + sq.slot * a.r_slot;
   const int keep = min(a.taps - 1, sq.len);
@@ -536,7 +543,7 @@ CAKE_API int cake_mixer_delta_prefill(int dt, const void* proj, long long ldp, c
               norm_w, 64 * ni, qn, kn, vv, tp, gm, o, state, ring, s_slot, r_slot, row_pos,
               row_slot, row_seq0, (const SeqRow*)seq, (const int2*)chunk, chunk0, NC, out, ldo};
   const dim3 gp((unsigned)(((long long)NC * (2 * G + H) + 3) / 4));
-  const dim3 gs((vdim + 15) / 16, H, B);
+  const dim3 gs(H, (vdim + 15) / 16, B);
   const dim3 go((unsigned)(((long long)N * H + 3) / 4));
   const int widest = 64 * ni > vdim ? 64 * ni : vdim;
   const int vec = dim % 2 == 0 && vdim % 2 == 0 && ldp % 2 == 0 && ((uintptr_t)proj % 4) == 0;

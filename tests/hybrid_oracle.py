@@ -25,16 +25,14 @@ def norm_around_one(x, w, eps):
 def rotate_pairs(x, dims, base, pos0=0):
     """x [T, heads, d]: neighbours (2i, 2i+1) of the first `dims` dimensions turn by
     p * base^(-2i/dims); the other dimensions pass."""
-    T = x.shape[0]
     out = x.clone()
+    p = torch.arange(pos0, pos0 + x.shape[0], dtype=torch.float64)
     for i in range(dims // 2):
-        f = base ** (-2.0 * i / dims)
-        for t in range(T):
-            a = (pos0 + t) * f
-            c, s = math.cos(a), math.sin(a)
-            u, v = x[t, :, 2 * i], x[t, :, 2 * i + 1]
-            out[t, :, 2 * i] = u * c - v * s
-            out[t, :, 2 * i + 1] = v * c + u * s
+        a = p * base ** (-2.0 * i / dims)
+        c, s = a.cos().to(x.dtype)[:, None], a.sin().to(x.dtype)[:, None]
+        u, v = x[:, :, 2 * i], x[:, :, 2 * i + 1]
+        out[:, :, 2 * i] = u * c - v * s
+        out[:, :, 2 * i + 1] = v * c + u * s
     return out
 
 
