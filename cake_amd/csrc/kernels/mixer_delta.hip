@@ -40,11 +40,11 @@ struct DeltaArgs {
   const float* dt_bias;   // [H] f32
   const float* norm_w;    // [vdim] f32
   int DR;                 // dim padded to 64
-  float* qn;              // [N][G][DR], zeros past dim
-  float* kn;              // [N][G][DR]
-  float* vv;              // [N][H][vdim]
+  float* qn;              // [N + 15][G][DR], zeros past dim
+  float* kn;              // [N + 15][G][DR]
+  float* vv;              // [N + 15][H][vdim]
   float* tp;              // [NC][H][2][16][16]: T, P
-  float* gm;              // [NC][H][16][4]: g_i, beta_i, G_15,i, g_15
+  float* gm;              // [NC][H][4][16]: g_i, beta_i, G_15,i, g_15
   float* o;               // [N][H][vdim]
   float* state;
   float* ring;
@@ -159,6 +159,9 @@ __global__ __launch_bounds__(256) void mixer_delta_prep_kernel(DeltaArgs a, int 
 #pragma unroll
       for (int e = 0; e < CPL; ++e)
         if (c0 + e < osize) o[e] = y[e] * r;
+    } else if (n0 + cnt == a.N) {  // the scan reads whole chunks: zeros past the last row
+      for (int e = 0; e < CPL; ++e)
+        if (c0 + e < osize) out[(long long)(n0 + t) * ostride + c0 + e] = 0.f;
     }
   }
 }
@@ -214,8 +217,8 @@ __global__ __launch_bounds__(256) void mixer_delta_chunk_kernel(DeltaArgs a) {
       float* tp = a.tp + ((long long)ch * a.H + h) * 512 + c;
 #pragma unroll
       for (int i = 0; i < 16; ++i) { tp[16 * i] = t[i]; tp[256 + 16 * i] = p[i]; }
-      *reinterpret_cast<float4*>(a.gm + (((long long)ch * a.H + h) * 16 + c) * 4) =
-          make_float4(expf(pre), beta, expf(suf), expf(all));
+      float* gp = a.gm + ((long long)ch * a.H + h) * 64 + c;
+      gp[0] = expf(pre); gp[16] = beta; gp[32] = expf(suf); gp[48] = expf(all);
     }
     __builtin_amdgcn_wave_barrier();
   }
@@ -224,8 +227,8 @@ __global__ __launch_bounds__(256) void mixer_delta_chunk_kernel(DeltaArgs a) {
 // One chunk's operands of a scan lane.
 template <int NI> struct ScanSet {
   u32x4 kp[NI], qp[NI], t, p;
-  float kt[NI][4], v[4];
-  cf32x4 gm[4];
+  float kt[NI][4], v[4], g15;
+  cf32x4 gi, beta, ge;  // tokens 4 g .. 4 g + 3
 };
 
 // grid (H, ceil(vdim / 16), B) — the column blocks of a head land on one XCD and share its
@@ -251,32 +254,45 @@ __global__ __launch_bounds__(256) void mixer_delta_scan_kernel(DeltaArgs a) {
       S[i][e] = sq.pos0 > 0 && cok && r < a.dim ? st[(long long)r * a.EP + col] : 0.f;
     }
   const int nc = (sq.len + kChunk - 1) / kChunk, ch0 = a.chunk0[blockIdx.z];
-  const int last = sq.row0 + sq.len - 1;
-  const int vcol = cok ? col : 0;
-
-  // rows past the end repeat the last (their beta is zero)
+  // A chunk's operands: a uniform base that moves with the chunk plus a lane offset that does
+  // not.  Rows past a sequence's end are another sequence's or zeros (prep) and count nothing:
+  // their beta is zero.
+  const unsigned krow = (unsigned)a.G * DR, vrow = (unsigned)a.H * a.vdim;
+  const unsigned koff = l15 * krow + r0 + 4 * g, toff = 16 * l15 + 4 * g;
+  unsigned ktoff[4], voff[4];
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    ktoff[e] = (4 * g + e) * krow + r0 + l15;
+    voff[e] = (4 * g + e) * vrow + (cok ? col : 0);
+  }
+  const float* kbase = a.kn + ((long long)sq.row0 * a.G + gh) * DR;
+  const float* qbase = a.qn + ((long long)sq.row0 * a.G + gh) * DR;
+  const float* vbase = a.vv + (long long)sq.row0 * vrow + (long long)h * a.vdim;
+  const float* tbase = a.tp + ((long long)ch0 * a.H + h) * 512;
+  const float* gbase = a.gm + ((long long)ch0 * a.H + h) * 64;
   auto load = [&](ScanSet<NI>& s, int c) __attribute__((always_inline)) {
-    const int n = sq.row0 + kChunk * c;
-    const long long nr = min(n + l15, last);
-    const float* kr = a.kn + (nr * a.G + gh) * DR + r0 + 4 * g;
-    const float* qr = a.qn + (nr * a.G + gh) * DR + r0 + 4 * g;
+    const float* kb = kbase + (long long)c * kChunk * krow;
+    const float* qb = qbase + (long long)c * kChunk * krow;
+    const float* vb = vbase + (long long)c * kChunk * vrow;
+    const float* tb = tbase + (long long)c * a.H * 512;
+    const float* gb = gbase + (long long)c * a.H * 64;
 #pragma unroll
     for (int i = 0; i < NI; ++i) {
-      s.kp[i] = *reinterpret_cast<const u32x4*>(kr + 16 * i);
-      s.qp[i] = *reinterpret_cast<const u32x4*>(qr + 16 * i);
+      s.kp[i] = *reinterpret_cast<const u32x4*>(kb + koff + 16 * i);
+      s.qp[i] = *reinterpret_cast<const u32x4*>(qb + koff + 16 * i);
     }
-    const float* tp = a.tp + ((long long)(ch0 + c) * a.H + h) * 512 + 16 * l15 + 4 * g;
-    s.t = *reinterpret_cast<const u32x4*>(tp);
-    s.p = *reinterpret_cast<const u32x4*>(tp + 256);
-    const float* gp = a.gm + (((long long)(ch0 + c) * a.H + h) * 16 + 4 * g) * 4;
 #pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      const long long nt = min(n + 4 * g + e, last);
-      s.gm[e] = *reinterpret_cast<const cf32x4*>(gp + 4 * e);
-      s.v[e] = a.vv[(nt * a.H + h) * a.vdim + vcol];
+    for (int e = 0; e < 4; ++e) s.v[e] = vb[voff[e]];
+    s.gi = *reinterpret_cast<const cf32x4*>(gb + 4 * g);
+    s.beta = *reinterpret_cast<const cf32x4*>(gb + 16 + 4 * g);
+    s.t = *reinterpret_cast<const u32x4*>(tb + toff);
+    s.ge = *reinterpret_cast<const cf32x4*>(gb + 32 + 4 * g);
+    s.g15 = gb[48];
 #pragma unroll
-      for (int i = 0; i < NI; ++i) s.kt[i][e] = a.kn[(nt * a.G + gh) * DR + r0 + 16 * i + l15];
-    }
+    for (int i = 0; i < NI; ++i)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) s.kt[i][e] = kb[ktoff[e] + 16 * i];
+    s.p = *reinterpret_cast<const u32x4*>(tb + 256 + toff);
   };
   auto chunk = [&](const ScanSet<NI>& s, int c) __attribute__((always_inline)) {
     const int buf = c & 1;
@@ -297,24 +313,24 @@ __global__ __launch_bounds__(256) void mixer_delta_scan_kernel(DeltaArgs a) {
     for (int w = 1; w < 4; ++w) ks += *reinterpret_cast<const cf32x4*>(ex[buf][w][0][lane]);
     cf32x4 rhs;
 #pragma unroll
-    for (int e = 0; e < 4; ++e) rhs[e] = s.gm[e][1] * (s.v[e] - s.gm[e][0] * ks[e]);
+    for (int e = 0; e < 4; ++e) rhs[e] = s.beta[e] * (s.v[e] - s.gi[e] * ks[e]);
     const cf32x4 u = mm_piece<kF32>(__builtin_bit_cast(uint4, s.t), __builtin_bit_cast(uint4, rhs),
                                     cf32x4{0.f, 0.f, 0.f, 0.f});
     cf32x4 ud;
 #pragma unroll
-    for (int e = 0; e < 4; ++e) ud[e] = s.gm[e][2] * u[e];
+    for (int e = 0; e < 4; ++e) ud[e] = s.ge[e] * u[e];
     const uint4 ub = __builtin_bit_cast(uint4, ud);
 #pragma unroll
     for (int i = 0; i < NI; ++i) {
       const cf32x4 ka = {s.kt[i][0], s.kt[i][1], s.kt[i][2], s.kt[i][3]};
-      S[i] = mm_piece<kF32>(__builtin_bit_cast(uint4, ka), ub, S[i] * s.gm[0][3]);
+      S[i] = mm_piece<kF32>(__builtin_bit_cast(uint4, ka), ub, S[i] * s.g15);
     }
     if (wave == (c & 3)) {  // the read-outs of a chunk: the waves take turns
       qs = *reinterpret_cast<const cf32x4*>(ex[buf][0][1][lane]);
 #pragma unroll
       for (int w = 1; w < 4; ++w) qs += *reinterpret_cast<const cf32x4*>(ex[buf][w][1][lane]);
 #pragma unroll
-      for (int e = 0; e < 4; ++e) qs[e] *= s.gm[e][0];
+      for (int e = 0; e < 4; ++e) qs[e] *= s.gi[e];
       const cf32x4 o = mm_piece<kF32>(__builtin_bit_cast(uint4, s.p), __builtin_bit_cast(uint4, u), qs);
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
@@ -327,6 +343,9 @@ __global__ __launch_bounds__(256) void mixer_delta_scan_kernel(DeltaArgs a) {
   ScanSet<NI> s0, s1;
   load(s0, 0);
   load(s1, min(1, nc - 1));
+  // once: with loads pending on the way in, the compiler waits for the newest loads in every
+  // round (its counts cover both ways into the loop)
+  __builtin_amdgcn_s_waitcnt(vm_wait(0));
   for (int c = 0; c < nc; c += 2) {
     chunk(s0, c);
     if (c + 1 >= nc) break;

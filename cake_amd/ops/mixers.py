@@ -338,7 +338,9 @@ def delta_prompt(sh: DeltaShape, proj, ab, rows: Rows, eps: float, conv, a_log, 
     abp, ldab = _mat(ab, "ab", f, N, 2 * sh.heads)
     op, ldo = _mat(out, "out", proj.dtype, N, sh.out_cols)
     G, H, NC, DR = sh.kv_heads, sh.heads, rows.chunk.shape[0], pad_to(sh.dim, 64)
-    sizes = (N * G * DR, N * G * DR, N * H * sh.vdim, NC * H * 512, NC * H * 64, N * H * sh.vdim)
+    NP = N + CHUNK - 1  # the scan reads whole chunks
+    sizes = (NP * G * DR, NP * G * DR, NP * H * sh.vdim, NC * H * 512, NC * H * 64,
+             N * H * sh.vdim)
     ws = torch.empty(sum(pad_to(s, 4) for s in sizes), device=dev, dtype=f)
     ptrs, o = [], 0
     for s in sizes:
