@@ -7,7 +7,7 @@
 // of both kernels then take 16-byte / 8-byte pieces of contiguous memory as their MFMA
 // operands, and no kernel transposes values in LDS.
 //
-//   * mixer_prep_qk / mixer_prep_v: prompt rows — rotation + norm of q and k, cache write.
+//   * mixer_prep: prompt rows — rotation + norm of q and k, cache write.
 //   * mixer_flash: prompt attention over a ragged batch.  S^T = K Q^T and O^T += V^T P^T
 //     (an accumulator of the first is the B operand of the second), 4 waves x 32 query
 //     rows, key tiles staged in LDS (double-buffered, next tile's loads in flight behind
@@ -49,13 +49,34 @@ __device__ __forceinline__ float lanes_sum(float v, int lph) {
   return v;
 }
 
+// values -> V^T: a wave takes 64 rows x 8 dims, so its stores run along the positions
+template <int DT>
+__device__ __forceinline__ void prep_v(const PrepArgs& a, int block) {
+  using E = typename St<DT>::E;
+  const int nrt = (a.N + 63) / 64, rt = block % nrt;
+  const int n = rt * 64 + (threadIdx.x & 63);
+  const int nch = (a.vdim + 7) / 8;
+  const int c = (block / nrt) * 4 + (threadIdx.x >> 6);
+  if (n >= a.N || c >= a.G * nch) return;
+  const int gh = c / nch, d0 = (c - gh * nch) * 8;
+  const E* src = reinterpret_cast<const E*>(a.proj) + (long long)n * a.ldp +
+                 (long long)(a.H + a.G) * a.dim + (long long)gh * a.vdim + d0;
+  E* dst = reinterpret_cast<E*>(a.vc) + a.row_slot[n] * a.v_slot +
+           ((long long)gh * a.DVP + d0) * a.S + a.row_pos[n];
+#pragma unroll
+  for (int e = 0; e < 8; ++e)
+    if (d0 + e < a.vdim) dst[(long long)e * a.S] = src[e];
+}
+
+// Blocks [0, nvb) move the values; the others take queries and keys:
 // lph lanes per (row, head), EPL consecutive dims each.  VEC: rows and heads on 2 EPL-byte
 // boundaries and dim % EPL == 0 (16-bit types).
 template <int DT, int EPL, bool VEC>
-__global__ __launch_bounds__(256) void mixer_prep_qk_kernel(PrepArgs a, int lph) {
+__global__ __launch_bounds__(256) void mixer_prep_kernel(PrepArgs a, int lph, int nvb) {
   using E = typename St<DT>::E;
+  if ((int)blockIdx.x < nvb) { prep_v<DT>(a, blockIdx.x); return; }
   const int per = 256 / lph;  // (row, head) items per workgroup
-  const int item = blockIdx.x * per + threadIdx.x / lph;
+  const int item = (blockIdx.x - nvb) * per + threadIdx.x / lph;
   const int l = threadIdx.x % lph, d0 = EPL * l;
   const int nh = a.H + a.G;
   const bool live = item < a.N * nh;  // lanes past the end shadow the last item
@@ -106,24 +127,6 @@ __global__ __launch_bounds__(256) void mixer_prep_qk_kernel(PrepArgs a, int lph)
       w[e] = (uint32_t)St<DT>::st(x[2 * e]) | ((uint32_t)St<DT>::st(x[2 * e + 1]) << 16);
     *reinterpret_cast<uint4*>(dst + d0) = make_uint4(w[0], w[1], w[2], w[3]);
   }
-}
-
-// values -> V^T: a wave takes 64 rows x 8 dims, so its stores run along the positions
-template <int DT>
-__global__ __launch_bounds__(256) void mixer_prep_v_kernel(PrepArgs a) {
-  using E = typename St<DT>::E;
-  const int n = blockIdx.x * 64 + (threadIdx.x & 63);
-  const int nch = (a.vdim + 7) / 8;
-  const int c = blockIdx.y * 4 + (threadIdx.x >> 6);
-  if (n >= a.N || c >= a.G * nch) return;
-  const int gh = c / nch, d0 = (c - gh * nch) * 8;
-  const E* src = reinterpret_cast<const E*>(a.proj) + (long long)n * a.ldp +
-                 (long long)(a.H + a.G) * a.dim + (long long)gh * a.vdim + d0;
-  E* dst = reinterpret_cast<E*>(a.vc) + a.row_slot[n] * a.v_slot +
-           ((long long)gh * a.DVP + d0) * a.S + a.row_pos[n];
-#pragma unroll
-  for (int e = 0; e < 8; ++e)
-    if (d0 + e < a.vdim) dst[(long long)e * a.S] = src[e];
 }
 
 // ---------------------------------------------------------------------------
@@ -677,12 +680,11 @@ CAKE_API int cake_mixer_prep(int dt, const void* proj, long long ldp, int N, int
   while (8 * lph < DP) lph <<= 1;  // <= 32
   const bool vec = dt != kF32 && dim % 8 == 0 && ldp % 8 == 0 && ((uintptr_t)proj % 16) == 0;
   const long long items = (long long)N * (H + G);
-  const dim3 g1((unsigned)((items + 256 / lph - 1) / (256 / lph)));
-  const dim3 g2((N + 63) / 64, (G * ((vdim + 7) / 8) + 3) / 4);
+  const int nvb = ((N + 63) / 64) * ((G * ((vdim + 7) / 8) + 3) / 4);
+  const dim3 g((unsigned)(nvb + (items + 256 / lph - 1) / (256 / lph)));
   CAKE_MIX_DT(dt, {
-    if (vec) hipLaunchKernelGGL((mixer_prep_qk_kernel<DT, 8, true>), g1, dim3(256), 0, st, a, lph);
-    else hipLaunchKernelGGL((mixer_prep_qk_kernel<DT, 8, false>), g1, dim3(256), 0, st, a, lph);
-    hipLaunchKernelGGL((mixer_prep_v_kernel<DT>), g2, dim3(256), 0, st, a);
+    if (vec) hipLaunchKernelGGL((mixer_prep_kernel<DT, 8, true>), g, dim3(256), 0, st, a, lph, nvb);
+    else hipLaunchKernelGGL((mixer_prep_kernel<DT, 8, false>), g, dim3(256), 0, st, a, lph, nvb);
   });
   return (int)hipGetLastError();
 }

@@ -114,9 +114,11 @@ __device__ __forceinline__ float row16_sum(float v) {
   return v;
 }
 
-// 32-bit gates and activations (the reciprocal is IEEE division, the exponential expf)
-__device__ __forceinline__ float sigmoid32(float x) { return 1.f / (1.f + expf(-x)); }
-__device__ __forceinline__ float silu32(float x) { return x / (1.f + expf(-x)); }
+// 32-bit gates and activations: the hardware exponential and reciprocal (1 ulp each)
+__device__ __forceinline__ float sigmoid32(float x) {
+  return __builtin_amdgcn_rcpf(1.f + __expf(-x));
+}
+__device__ __forceinline__ float silu32(float x) { return x * sigmoid32(x); }
 __device__ __forceinline__ float softplus32(float x) { return x > 20.f ? x : log1pf(expf(x)); }
 __device__ __forceinline__ float gelu_erf32(float x) {
   return 0.5f * x * (1.f + erff(x * 0.70710678118654752f));

@@ -76,11 +76,11 @@ __device__ __forceinline__ float conv_tap(const DeltaArgs& a, int n, int pos, in
 }
 
 constexpr int kChunk = 16;
-constexpr int kWin = 8;  // taps a lane keeps in registers
 
 // A wave per (chunk, unit): units [0, 2G) the q and k heads, [2G, 2G + H) the value heads;
-// CPL consecutive channels per lane, the last kWin inputs of each in registers.
-template <int DT, int CPL>
+// CPL consecutive channels per lane, the last kWin inputs of each in registers (longer
+// convolutions read the older ones from memory).
+template <int DT, int CPL, int kWin>
 __global__ __launch_bounds__(256) void mixer_delta_prep_kernel(DeltaArgs a, int vec) {
   using E = typename St<DT>::E;
   const int lane = threadIdx.x & 63;
@@ -166,28 +166,39 @@ __global__ __launch_bounds__(256) void mixer_delta_prep_kernel(DeltaArgs a, int 
   }
 }
 
-// grid (NC, G), 256 threads: the state-independent matrices of every head of a group
+// A wave per (chunk, kv head): the state-independent matrices of every head of the group
 __global__ __launch_bounds__(256) void mixer_delta_chunk_kernel(DeltaArgs a) {
-  __shared__ float kk[16][17], qk[16][17], am[16][16][17];
-  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, l15 = lane & 15, g = lane >> 4;
-  const int ch = blockIdx.x, gh = blockIdx.y;
+  __shared__ float kks[4][16][17], qks[4][16][17], ams[4][4][16][17];
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, l15 = lane & 15, g = lane >> 4;
+  const long long item = (long long)blockIdx.x * 4 + wave;
+  if (item >= (long long)a.NC * a.G) return;  // waves share nothing
+  const int ch = (int)(item / a.G), gh = (int)(item - (long long)ch * a.G);
   const int n0 = a.chunk[ch].x, cnt = a.chunk[ch].y;
-  if (wave < 2) {  // k.k and q.k: rows past the chunk's end repeat the last, masked below
+  float(&kk)[16][17] = kks[wave];
+  float(&qk)[16][17] = qks[wave];
+  float(&am)[4][16][17] = ams[wave];
+  {  // k.k and q.k: rows past the chunk's end repeat the last, masked below
     const int row = n0 + min(l15, cnt - 1);
     const float* kp = a.kn + ((long long)row * a.G + gh) * a.DR + 4 * g;
-    const float* xp = (wave == 0 ? a.kn : a.qn) + ((long long)row * a.G + gh) * a.DR + 4 * g;
-    cf32x4 acc{0.f, 0.f, 0.f, 0.f};
-    for (int d = 0; d < a.DR; d += 16)
-      acc = mm_piece<kF32>(*reinterpret_cast<const uint4*>(xp + d),
-                           *reinterpret_cast<const uint4*>(kp + d), acc);
+    const float* qp = a.qn + ((long long)row * a.G + gh) * a.DR + 4 * g;
+    cf32x4 ka{0.f, 0.f, 0.f, 0.f}, qa{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+    for (int d = 0; d < a.DR; d += 16) {  // DR % 64 == 0: four pieces of each in flight
+      const uint4 kv = *reinterpret_cast<const uint4*>(kp + d);
+      ka = mm_piece<kF32>(kv, kv, ka);
+      qa = mm_piece<kF32>(*reinterpret_cast<const uint4*>(qp + d), kv, qa);
+    }
 #pragma unroll
-    for (int e = 0; e < 4; ++e) (wave == 0 ? kk : qk)[4 * g + e][l15] = acc[e];
+    for (int e = 0; e < 4; ++e) {
+      kk[4 * g + e][l15] = ka[e];
+      qk[4 * g + e][l15] = qa[e];
+    }
   }
-  __syncthreads();
+  __builtin_amdgcn_wave_barrier();  // a wave's LDS accesses complete in order
   const int R = a.H / a.G;
-  for (int h0 = 0; h0 < R; h0 += 16) {
+  for (int h0 = 0; h0 < R; h0 += 4) {
     // sixteen lanes per head, lane c = column c (and token c)
-    const int hs = wave * 4 + g, hl = h0 + hs, h = gh * R + min(hl, R - 1), c = l15;
+    const int hs = g, hl = h0 + hs, h = gh * R + min(hl, R - 1), c = l15;
     const bool ok = c < cnt;
     const float* ab = a.ab + (long long)(n0 + min(c, cnt - 1)) * a.ldab;
     const float ld = ok ? fmaxf(-expf(a.a_log[h]) * softplus32(ab[h] + a.dt_bias[h]), -1e30f) : 0.f;
@@ -204,7 +215,7 @@ __global__ __launch_bounds__(256) void mixer_delta_chunk_kernel(DeltaArgs a) {
       am[hs][i][c] = i > c ? bi * gi * kk[i][c] : 0.f;
       p[i] = i >= c ? gi * qk[i][c] : 0.f;
     }
-    __builtin_amdgcn_wave_barrier();  // each head's matrix is one wave's own
+    __builtin_amdgcn_wave_barrier();
     // column c of (I + A)^-1 by forward substitution
 #pragma unroll
     for (int i = 0; i < 16; ++i) {
@@ -566,11 +577,18 @@ CAKE_API int cake_mixer_delta_prefill(int dt, const void* proj, long long ldp, c
   const dim3 go((unsigned)(((long long)N * H + 3) / 4));
   const int widest = 64 * ni > vdim ? 64 * ni : vdim;
   const int vec = dim % 2 == 0 && vdim % 2 == 0 && ldp % 2 == 0 && ((uintptr_t)proj % 4) == 0;
+#define CAKE_PREP1(CPL, W) \
+  hipLaunchKernelGGL((mixer_delta_prep_kernel<DT, CPL, W>), gp, dim3(256), 0, st, a, vec)
+#define CAKE_PREP(W)                        \
+  do {                                      \
+    if (widest <= 64) CAKE_PREP1(1, W);     \
+    else if (widest <= 128) CAKE_PREP1(2, W); \
+    else CAKE_PREP1(4, W);                  \
+  } while (0)
   CAKE_MIX_DT(dt, {
-    if (widest <= 64) hipLaunchKernelGGL((mixer_delta_prep_kernel<DT, 1>), gp, dim3(256), 0, st, a, vec);
-    else if (widest <= 128) hipLaunchKernelGGL((mixer_delta_prep_kernel<DT, 2>), gp, dim3(256), 0, st, a, vec);
-    else hipLaunchKernelGGL((mixer_delta_prep_kernel<DT, 4>), gp, dim3(256), 0, st, a, vec);
-    hipLaunchKernelGGL(mixer_delta_chunk_kernel, dim3(NC, G), dim3(256), 0, st, a);
+    if (taps <= 4) CAKE_PREP(4); else CAKE_PREP(8);
+    hipLaunchKernelGGL(mixer_delta_chunk_kernel, dim3((unsigned)(((long long)NC * G + 3) / 4)),
+                       dim3(256), 0, st, a);
     if (ni == 1) hipLaunchKernelGGL((mixer_delta_scan_kernel<DT, 1>), gs, dim3(256), 0, st, a);
     else if (ni == 2) hipLaunchKernelGGL((mixer_delta_scan_kernel<DT, 2>), gs, dim3(256), 0, st, a);
     else if (ni == 3) hipLaunchKernelGGL((mixer_delta_scan_kernel<DT, 3>), gs, dim3(256), 0, st, a);
