@@ -583,6 +583,55 @@ def test_generation_stops_and_samples(cuda, checkpoint):
     assert ids[0] == ids[1] and len(ids[0]) == 12
 
 
+def test_metrics_leave_the_state_alone(cuda, checkpoint):
+    """Per-layer timing between two tokens replays layers; the recurrent state comes back."""
+    m = _master(checkpoint, "bf16", "--temperature", "0")
+
+    def run(measure):
+        m.reset()
+        _prompt_ids(m.llm, "timing")
+        out = [m.llm.next_token(0).id]
+        for i in range(1, 16):
+            if measure and i == 8:
+                d = m.llm.metrics()
+                assert len(d["layer_ms"]) == len(m.llm.model.runs) and d["layers_ms_total"] > 0
+            out.append(m.llm.next_token(i).id)
+        return out
+    assert run(False) == run(True)
+
+
+def test_rest_api(cuda, checkpoint):
+    from fastapi.testclient import TestClient
+
+    from cake_amd.api.server import create_app
+    m = _master(checkpoint, "bf16", "--temperature", "0")
+    body = {"messages": [{"role": "user", "content": "hello"}], "max_tokens": 6}
+    with TestClient(create_app(m)) as c:
+        a, b = (c.post("/api/v1/chat/completions", json=body).json() for _ in range(2))
+    assert a["model"] == "fonapel" and a["choices"] == b["choices"]
+    assert 0 < a["usage"]["completion_tokens"] <= 6
+
+
+def test_cli_executable(cuda, checkpoint):
+    """The cake-cli executable hands the design to the embedded runtime and generates what the
+    master does."""
+    import os
+    import subprocess
+    root = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+    r = subprocess.run([os.path.join(root, "cake_amd", "lib", "cake-cli"), "--model",
+                        str(checkpoint), "--topology", "/nonexistent", "--dtype", "bf16",
+                        "--temperature", "0", "--prompt", "hi", "-n", "8", "--max-seq-len", "512"],
+                       capture_output=True, timeout=110, cwd=root)
+    assert r.returncode == 0, r.stderr.decode(errors="replace")[-2000:]
+    m = _master(checkpoint, "bf16", "--temperature", "0", "--prompt", "hi", "-n", "8")
+    from cake_amd.models.chat import Message
+    m.llm.add_message(Message.system(m.ctx.args.system_prompt))
+    m.llm.add_message(Message.user("hi"))
+    out = []
+    m.generate_text(out.append)
+    assert r.stdout.decode(errors="replace").strip("\n") == "".join(out).strip("\n")
+
+
 def test_graph_survives_pool_growth(cuda, checkpoint):
     """Steps of other sequences between two generations, with the pool moving: the decoder
     captures again and generates the same tokens."""

@@ -126,3 +126,16 @@ def test_native_bridge_tokenizer_matches_generator(ckpt):
     assert r["ids"] == list(ids) and r["eos"] == sorted(eos)
     for t in (5, 72, 300, 259):
         assert B.decode_token(json.dumps({"model": str(ckpt), "id": t})) == (gen._decode(t) or "")
+
+
+def test_cli_leaves_other_designs_to_the_embedded_runtime(tmp_path):
+    """A config.json that names a design is not the native engine's: the embedded registry
+    answers for it (here: an unknown one, and a placement it refuses)."""
+    (tmp_path / "config.json").write_text('{"architecture": "Nothing"}')
+    r = _run([CLI, "--model", str(tmp_path), "--topology", "/nonexistent", "-n", "1"])
+    assert r.returncode != 0 and "unknown architecture" in r.stderr
+    (tmp_path / "config.json").write_text('{"architecture": "Fonapel"}')
+    topo = tmp_path / "t.yml"
+    topo.write_text("w1:\n  host: '127.0.0.1:1'\n  layers: ['model.layers.0-1']\n")
+    r = _run([CLI, "--model", str(tmp_path), "--topology", str(topo), "-n", "1"])
+    assert r.returncode != 0 and "one GPU" in r.stderr
