@@ -1,1 +1,1 @@
-"""Model families: Llama-3 text generation and Stable Diffusion image generation."""
+"""Model families: Llama-3 and hybrid-design text generation, Stable Diffusion images."""

@@ -94,7 +94,7 @@ class DeviceDecoder:
         self.params.copy_(K.pack_sample_params(sampling))
 
     def profile_layers(self, reps: int = 3) -> list[float]:
-        """Per-layer decode kernel time (ms; SURVEY §5.5): each layer's five launches
+        """Per-layer decode kernel time (ms): each layer's five launches
         captured as its own small graph and replayed between timing events, at the
         current device position (the K/V row it writes is the next step's, which that
         step rewrites).  Run between generations (--metrics)."""

@@ -126,7 +126,7 @@ def test_gemm_alpha(cuda, alpha, M_, N, K):
 
 # ---------------------------------------------------------------------------- attention
 # heads, kv_heads, dim, vdim, rotated dims
-ATTN = [(4, 2, 64, 48, 16), (2, 2, 20, 20, 0), (3, 1, 66, 30, 66), (8, 2, 128, 128, 64),
+ATTN = [(4, 2, 64, 56, 24), (2, 2, 20, 20, 0), (3, 1, 66, 30, 66), (8, 2, 128, 128, 64),
         (20, 1, 64, 64, 64), (2, 1, 200, 72, 10), (2, 1, 40, 256, 40)]
 
 
@@ -283,7 +283,7 @@ def test_attention_portions_and_used_slots(cuda):
 
 # ---------------------------------------------------------------------------- delta rule
 # heads, kv_heads, dim, vdim, taps
-DELTA = [(2, 2, 32, 32, 4), (4, 2, 24, 40, 3), (3, 1, 20, 12, 1), (2, 1, 128, 128, 4),
+DELTA = [(2, 2, 40, 40, 4), (4, 2, 24, 40, 3), (3, 1, 20, 12, 1), (2, 1, 128, 128, 4),
          (2, 2, 200, 72, 2), (1, 1, 64, 250, 7), (2, 1, 256, 256, 4)]
 
 
